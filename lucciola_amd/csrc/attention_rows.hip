@@ -1,0 +1,109 @@
+// A prologue of the masked attention (masked_attention.hip) for layers whose queries and keys are normed as whole
+// rows: from a step's float32 projections q | k | v (side by side, heads of d, d and dv entries) it makes q for the
+// attention kernels and the rows of the cache.
+//   x <- proj + bias                                                           (bias, where given)
+//   q <- q / sqrt(mean of q^2 over ALL its heads' entries + eps) * q_weight    (where given; k likewise, on its own)
+//   rotation of the first `rot` entries of every q and k head: entry i with i + rot / 2 (half), or 2i with 2i + 1
+//   v is left in values_out as it is (where given), then v <- (1 - mix) v + mix mix_from    (where mix_from is given)
+// Everything is float32; q, k and v are rounded once, to the type of the cache.  Keys lie token-major, values
+// transposed inside their page.
+#include "common.h"
+
+namespace lc {
+
+constexpr int AR_THREADS = 256;
+
+// grid (tokens, parts): every part of a token sums the whole rows and writes its share of the entries.
+template <typename T>
+__global__ __launch_bounds__(AR_THREADS) void attention_rows_kernel(
+    const float* __restrict__ proj, int cols, int nq, int nk, int nv, int d, int dv, const float* __restrict__ bias,
+    const float* __restrict__ q_weight, const float* __restrict__ k_weight, float eps, const float* __restrict__ table,
+    int rot, int half, const int* __restrict__ positions, const float* __restrict__ mix_from, float mix,
+    float* __restrict__ values_out, T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache,
+    const int* __restrict__ rows, int page_size) {
+    __shared__ float scratch[16];
+    const int t = blockIdx.x;
+    const float* x = proj + (size_t)t * cols;
+    const int q_cols = nq * d, qk_cols = (nq + nk) * d, v_cols = nv * dv;
+    float by_q = 1.f, by_k = 1.f;
+    if (q_weight) {             // the same condition in every thread
+        float qq = 0.f, kk = 0.f;
+        for (int c = threadIdx.x; c < qk_cols; c += AR_THREADS) {
+            const float v = bias ? x[c] + bias[c] : x[c];
+            if (c < q_cols) qq = fmaf(v, v, qq);
+            else kk = fmaf(v, v, kk);
+        }
+        by_q = 1.f / sqrtf(block_sum(qq, scratch) / (float)q_cols + eps);
+        by_k = 1.f / sqrtf(block_sum(kk, scratch) / (float)(nk * d) + eps);
+    }
+    const int turned = table ? rot / 2 : 0;          // pairs of a head that are rotated
+    const int units = d - turned;                    // pairs and single entries of a head
+    const float* angle = table ? table + (size_t)positions[t] * rot : nullptr;
+    const int slot = rows ? rows[t] : -1;
+    const int page = slot >= 0 ? slot / page_size : 0, place = slot >= 0 ? slot % page_size : 0;
+    auto normed = [&](int c) {
+        float v = bias ? x[c] + bias[c] : x[c];
+        if (q_weight) v = c < q_cols ? v * by_q * q_weight[c] : v * by_k * k_weight[c - q_cols];
+        return v;
+    };
+    auto put = [&](int c, float v) {
+        if (c < q_cols) q_out[(size_t)t * q_cols + c] = from_f32<T>(v);
+        else if (slot >= 0) k_cache[(size_t)slot * nk * d + (c - q_cols)] = from_f32<T>(v);
+    };
+    const int qk_units = (nq + nk) * units;
+    for (int idx = blockIdx.y * AR_THREADS + threadIdx.x; idx < qk_units + v_cols; idx += gridDim.y * AR_THREADS) {
+        if (idx < qk_units) {
+            const int head = idx / units, u = idx - head * units, base = head * d;
+            if (u < turned) {
+                const int c0 = base + (half ? u : 2 * u), c1 = base + (half ? u + turned : 2 * u + 1);
+                const float a = normed(c0), b = normed(c1), cs = angle[u], sn = angle[turned + u];
+                put(c0, a * cs - b * sn);
+                put(c1, fmaf(b, cs, a * sn));
+            } else {
+                const int c = base + u + turned;
+                put(c, normed(c));
+            }
+        } else {
+            const int e = idx - qk_units;
+            float v = bias ? x[qk_cols + e] + bias[qk_cols + e] : x[qk_cols + e];
+            if (values_out) values_out[(size_t)t * v_cols + e] = v;
+            if (mix_from) v = fmaf(mix, mix_from[(size_t)t * v_cols + e], (1.f - mix) * v);
+            if (slot >= 0) v_cache[((size_t)page * v_cols + e) * page_size + place] = from_f32<T>(v);
+        }
+    }
+}
+
+}  // namespace lc
+
+using namespace lc;
+
+LC_API int lc_attention_rows(const float* proj, int cols, int T, int nq, int nk, int nv, int d, int dv, const float* bias,
+                             const float* q_weight, const float* k_weight, float eps, const float* table, int rot,
+                             int half, const int* positions, const float* mix_from, float mix, float* values_out,
+                             void* q_out, void* k_cache, void* v_cache, int dt, const int* rows, int page_size,
+                             hipStream_t stream) {
+    LC_CHECK(T >= 0 && nq > 0 && nk > 0 && nv > 0 && d > 0 && dv > 0 && cols >= (nq + nk) * d + nv * dv,
+             "attention rows: bad sizes");
+    if (T == 0) return 0;
+    LC_CHECK(proj && q_out, "attention rows: null pointer");
+    LC_CHECK((q_weight == nullptr) == (k_weight == nullptr), "attention rows: q and k are normed together");
+    LC_CHECK(!table || (rot > 0 && rot % 2 == 0 && rot <= d && positions), "attention rows: bad rotation");
+    LC_CHECK(!rows || (k_cache && v_cache && page_size > 0), "attention rows: rows without a cache");
+    // few tokens: several workgroups a token, so that the card is not left to a handful of them
+    const int total = (nq + nk) * d + nv * dv;
+    int parts = 1;
+    while (parts < 8 && T * parts * 2 <= device_cus() && parts * 2 * AR_THREADS <= total) parts *= 2;
+    const dim3 grid(T, parts);
+    if (dt == DT_F32)
+        attention_rows_kernel<float><<<grid, AR_THREADS, 0, stream>>>(
+            proj, cols, nq, nk, nv, d, dv, bias, q_weight, k_weight, eps, table, rot, half, positions, mix_from, mix,
+            values_out, (float*)q_out, (float*)k_cache, (float*)v_cache, rows, page_size);
+    else if (dt == DT_BF16)
+        attention_rows_kernel<bf16><<<grid, AR_THREADS, 0, stream>>>(
+            proj, cols, nq, nk, nv, d, dv, bias, q_weight, k_weight, eps, table, rot, half, positions, mix_from, mix,
+            values_out, (bf16*)q_out, (bf16*)k_cache, (bf16*)v_cache, rows, page_size);
+    else
+        LC_CHECK(false, "attention rows: unknown dtype %d", dt);
+    LC_LAUNCH_CHECK("attention_rows");
+    return 0;
+}

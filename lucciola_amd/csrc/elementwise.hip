@@ -58,12 +58,14 @@ __global__ void embedding_kernel(const int* __restrict__ ids, const TW* __restri
 // With sumsq: out[r] = v * w and sumsq[r] = sum(v^2): the row's factor is left to the product
 // that reads out (gemm_bf16.hip, scaled rows).
 // With shares > 0, delta is not a tensor of T but float32 [shares][all rows of h][n]: the shares
-// of a product that was cut along K (gemm_bf16.hip), added here in their order.
+// of a product that was cut along K (gemm_bf16.hip), added here in their order.  bias [n] (or
+// null): the branch's own, added to every row of delta.
 template <typename T>
 __global__ void rmsnorm_kernel(float* __restrict__ h, const T* __restrict__ delta,
                                const int* __restrict__ rows, const float* __restrict__ w,
                                float eps, T* __restrict__ out, int n, int write_h,
-                               float* __restrict__ sumsq, int shares, size_t share_stride) {
+                               float* __restrict__ sumsq, int shares, size_t share_stride,
+                               const float* __restrict__ bias) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
     const int src = rows ? rows[r] : r;
@@ -71,10 +73,11 @@ __global__ void rmsnorm_kernel(float* __restrict__ h, const T* __restrict__ delt
     const T* dr = (delta && !shares) ? delta + (size_t)src * n : nullptr;
     const float* pr = shares ? reinterpret_cast<const float*>(delta) + (size_t)src * n : nullptr;
     auto branch = [&](int i) {
-        if (dr) return to_f32(dr[i]);
+        const float b = bias ? bias[i] : 0.f;
+        if (dr) return to_f32(dr[i]) + b;
         float t = 0.f;
         for (int s = 0; s < shares; ++s) t += pr[s * share_stride + i];
-        return t;
+        return t + b;
     };
     float ss = 0.f;
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
@@ -122,7 +125,7 @@ template <typename T, int THREADS, int CHUNKS>
 __global__ __launch_bounds__(THREADS) void rmsnorm_vec_kernel(
     float* __restrict__ h, const T* __restrict__ delta, const int* __restrict__ rows,
     const float* __restrict__ w, float eps, T* __restrict__ out, int n, int write_h,
-    float* __restrict__ sumsq, int shares, size_t share_stride) {
+    float* __restrict__ sumsq, int shares, size_t share_stride, const float* __restrict__ bias) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
     const int src = rows ? rows[r] : r;
@@ -140,6 +143,17 @@ __global__ __launch_bounds__(THREADS) void rmsnorm_vec_kernel(
             hv[c] = *reinterpret_cast<const Pack8<float>*>(hr + chunk * 8);
             if (dr) dv[c] = *reinterpret_cast<const Pack8<T>*>(dr + chunk * 8);
             wv[c] = *reinterpret_cast<const Pack8<float>*>(w + chunk * 8);
+        }
+    }
+    if (bias) {
+#pragma unroll
+        for (int c = 0; c < CHUNKS; ++c) {
+            const int chunk = threadIdx.x + c * THREADS;
+            if (chunk < chunks) {
+                const Pack8<float> bv = *reinterpret_cast<const Pack8<float>*>(bias + chunk * 8);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) hv[c].set(i, hv[c].get(i) + bv.get(i));
+            }
         }
     }
     if (pr) {   // the shares of the branch's product, in their order, then the stream
@@ -428,7 +442,8 @@ LC_API int lc_embedding(const int* ids, const void* table, int table_dt, float* 
 // is added to h is their sum in the order of the shares.
 LC_API int lc_rmsnorm(float* h, const void* delta, const int* rows, const float* w, float eps,
                       void* out, int dt, int R, int n, int write_h, float* sumsq, int shares,
-                      int h_rows, hipStream_t stream) {
+                      int h_rows, const float* bias, hipStream_t stream) {
+    LC_CHECK(!bias || delta, "rmsnorm: a branch's bias without the branch");
     LC_CHECK(shares >= 0 && (shares == 0 || (delta && h_rows > 0)), "rmsnorm: bad shares %d", shares);
     const size_t share_stride = (size_t)h_rows * n;
     LC_CHECK(R >= 0 && n > 0, "rmsnorm: bad sizes R=%d n=%d", R, n);
@@ -438,27 +453,27 @@ LC_API int lc_rmsnorm(float* h, const void* delta, const int* rows, const float*
     const int threads = n >= 1024 ? 256 : (n >= 256 ? 128 : 64);
     const bool vec = n % 8 == 0 && n >= 512 && n <= RN_THREADS * RN_CHUNKS * 8 &&
                      (uintptr_t)h % 16 == 0 && (uintptr_t)delta % 16 == 0 && (uintptr_t)out % 16 == 0 &&
-                     (uintptr_t)w % 16 == 0;
+                     (uintptr_t)w % 16 == 0 && (uintptr_t)bias % 16 == 0;
     // float32 results must not depend on how many rows share a step: there the shape of the
     // kernel, and with it the grouping of a row's sum of squares, follows from n alone
     const bool few = dt == DT_BF16 && R <= 128 && n > 2048 && n <= 8192;
     if (dt == DT_F32) {
         if (vec)
             rmsnorm_vec_kernel<float, RN_THREADS, RN_CHUNKS><<<R, RN_THREADS, 0, stream>>>(h, (const float*)delta, rows, w, eps,
-                                                                    (float*)out, n, write_h, sumsq, shares, share_stride);
+                                                                    (float*)out, n, write_h, sumsq, shares, share_stride, bias);
         else
             rmsnorm_kernel<float><<<R, threads, 0, stream>>>(h, (const float*)delta, rows, w, eps,
-                                                             (float*)out, n, write_h, sumsq, shares, share_stride);
+                                                             (float*)out, n, write_h, sumsq, shares, share_stride, bias);
     } else if (dt == DT_BF16) {
         if (vec && few)
             rmsnorm_vec_kernel<bf16, 1024, 1><<<R, 1024, 0, stream>>>(h, (const bf16*)delta, rows, w, eps,
-                                                                      (bf16*)out, n, write_h, sumsq, shares, share_stride);
+                                                                      (bf16*)out, n, write_h, sumsq, shares, share_stride, bias);
         else if (vec)
             rmsnorm_vec_kernel<bf16, RN_THREADS, RN_CHUNKS><<<R, RN_THREADS, 0, stream>>>(h, (const bf16*)delta, rows, w, eps,
-                                                                   (bf16*)out, n, write_h, sumsq, shares, share_stride);
+                                                                   (bf16*)out, n, write_h, sumsq, shares, share_stride, bias);
         else
             rmsnorm_kernel<bf16><<<R, threads, 0, stream>>>(h, (const bf16*)delta, rows, w, eps,
-                                                            (bf16*)out, n, write_h, sumsq, shares, share_stride);
+                                                            (bf16*)out, n, write_h, sumsq, shares, share_stride, bias);
     } else {
         LC_CHECK(false, "rmsnorm: unknown dtype %d", dt);
     }

@@ -45,11 +45,20 @@ template <int CTRL> __device__ __forceinline__ float lane_swap(float v) {
     return __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), CTRL, 0xF, 0xF, true));
 }
 
-// silu(g) * u with silu(g) = g / (1 + exp(-g))   (reference: src/kernels/swiglu.cu:8,31-35).
+// What the gated epilogue makes of a gate and an up entry: with g' = min(g, limit) and u' = u held inside
+// -limit .. limit, g' sigmoid(slope g') (u' + shift).  No limit, slope 1 and shift 0 is silu(g) u (reference:
+// src/kernels/swiglu.cu:8,31-35), to the bit.
+struct GateForm {
+    float limit, slope, shift;
+};
+static constexpr GateForm kSilu{INFINITY, 1.f, 0.f};
+
 // exp and the reciprocal are the hardware's single instructions (about one unit in the last
 // place each); the results of these products are rounded to bfloat16 afterwards.
-__device__ __forceinline__ float swiglu_f(float g, float u) {
-    return g * __builtin_amdgcn_rcpf(1.f + __expf(-g)) * u;
+__device__ __forceinline__ float gated_f(float g, float u, GateForm form) {
+    g = fminf(g, form.limit);
+    u = fminf(fmaxf(u, -form.limit), form.limit);
+    return g * __builtin_amdgcn_rcpf(1.f + __expf(-form.slope * g)) * (u + form.shift);
 }
 
 typedef __attribute__((address_space(3))) void* lds_ptr_t;
@@ -78,6 +87,8 @@ struct SkinnyFuse {
     bf16* next_x;
     float* next_partials;
     int stride;
+    const float* resid_bias;    // epilogue 2: a bias [N] that every row of the product gets, or null
+    GateForm form;              // epilogue 1
 };
 constexpr int SK_MAX_PIECES = 512;   // pieces of a sum of squares that a SCALE product reads
 
@@ -182,6 +193,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const bf16* __r
             for (int nt = 0; nt < NT; ++nt) {
                 const bool mine = g == 0 && r < M && e_n + nt * 16 < n_end;
                 e_resid[nt] = mine ? fuse.resid[(size_t)r * N + e_n + nt * 16] : 0.f;
+                if (mine && fuse.resid_bias) e_resid[nt] += fuse.resid_bias[e_n + nt * 16];
                 e_w[nt] = mine ? fuse.next_w[e_n + nt * 16] : 0.f;
             }
         }
@@ -292,7 +304,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const bf16* __r
                         const int n = e_n + nt * 16;
                         const int col = (n >> 4) * 8 + (n & 7);
                         if (g == 0 && r < M && n < n_end)
-                            store_out<TO>(out + (size_t)r * (N / 2) + col, swiglu_f(gate * factor, up * factor));
+                            store_out<TO>(out + (size_t)r * (N / 2) + col, gated_f(gate * factor, up * factor, fuse.form));
                     }
                 }
             }
@@ -466,6 +478,7 @@ __global__ __launch_bounds__(1024) void gemm_runs_kernel(const bf16* __restrict_
         acc = floatx4{0.f, 0.f, 0.f, 0.f};
         if (EPI == 2 && threadIdx.x < 256 && e_m < M && n0 + e_j < n_end) {
             e_resid = fuse.resid[(size_t)e_m * N + n0 + e_j];
+            if (fuse.resid_bias) e_resid += fuse.resid_bias[n0 + e_j];
             e_w = fuse.next_w[n0 + e_j];
         }
     };
@@ -526,7 +539,7 @@ __global__ __launch_bounds__(1024) void gemm_runs_kernel(const bf16* __restrict_
             } else if (EPI == 1) {
                 // rows of w come in blocks of 16: 8 gate rows, then their 8 up rows; out has N / 2 columns
                 if (mine && e_j < 8)
-                    store_out<TO>(out + (size_t)e_m * (N / 2) + (n >> 4) * 8 + (n & 7), swiglu_f(t * factor, t_up * factor));
+                    store_out<TO>(out + (size_t)e_m * (N / 2) + (n >> 4) * 8 + (n & 7), gated_f(t * factor, t_up * factor, fuse.form));
             } else {
                 float sq = 0.f;
                 if (mine) {
@@ -608,7 +621,8 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(const bf16* __
                                                          const bf16* __restrict__ w,
                                                          TO* __restrict__ out, float* __restrict__ part,
                                                          int M, int N, int K, int tiles_m, int tile_base,
-                                                         int tile_count, int compact, int skew_step) {
+                                                         int tile_count, int compact, int skew_step,
+                                                         GateForm form) {
     // WM x WN waves, each owning (BM / WM) x (BN / WN) of the tile as TM x TN products of 32 x 32
     constexpr int S = TL_STAGES;
     constexpr int NW = WM * WN;
@@ -838,7 +852,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(const bf16* __
                     float first = acc[i][j][v], second = acc[i][j][v + 1];
                     asm volatile("" : "+v"(first), "+v"(second));   // two values, not one indexed by `up`
                     const float got = lane_swap<0x128>(up ? first : second);   // lane ^ 8
-                    const float r = swiglu_f(up ? got : first, up ? second : got);
+                    const float r = gated_f(up ? got : first, up ? second : got, form);
                     const int dm = i * 32 + (v >> 2) * 8 + (v & 3);
                     if (mrow + (up ? 1 : 0) + dm < M && ng + j * 32 < N)
                         store_out<TO>(dst + (size_t)dm * (N / 2) + j * 16, r);
@@ -888,7 +902,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(const bf16* __
 // out = sum over the shares of part[s][M][N], added in the order of s; EPI as in the products
 template <int EPI, typename TO>
 __global__ void splitk_reduce_kernel(const float* __restrict__ part, TO* __restrict__ out, int M, int N,
-                                     int S) {
+                                     int S, GateForm form) {
     const size_t MN = (size_t)M * N;
     if (EPI == 0) {
         for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < MN;
@@ -906,7 +920,7 @@ __global__ void splitk_reduce_kernel(const float* __restrict__ part, TO* __restr
             const size_t gi = m * N + (size_t)(c >> 3) * 16 + (c & 7);
             float g = 0.f, u = 0.f;
             for (int s = 0; s < S; ++s) { g += part[s * MN + gi]; u += part[s * MN + gi + 8]; }
-            store_out<TO>(out + idx, swiglu_f(g, u));
+            store_out<TO>(out + idx, gated_f(g, u, form));
         }
     }
 }
@@ -917,7 +931,7 @@ __global__ void splitk_reduce_kernel(const float* __restrict__ part, TO* __restr
 template <int EPI, typename TO>
 __global__ __launch_bounds__(256) void tail_reduce_kernel(const float* __restrict__ part, TO* __restrict__ out,
                                                           int M, int N, int BM, int BN, int tiles_m,
-                                                          int tile_base, int count, int S) {
+                                                          int tile_base, int count, int S, GateForm form) {
     const int local = blockIdx.x, tile = tile_base + local;
     const int m0 = (tile % tiles_m) * BM, n0 = (tile / tiles_m) * BN;
     const size_t area = (size_t)BM * BN;
@@ -936,7 +950,7 @@ __global__ __launch_bounds__(256) void tail_reduce_kernel(const float* __restric
                 g += src[(size_t)s * count * area + e];
                 u += src[(size_t)s * count * area + e + 8];
             }
-            store_out<TO>(out + (size_t)m * (N / 2) + (size_t)(n >> 4) * 8 + (n & 7), swiglu_f(g, u));
+            store_out<TO>(out + (size_t)m * (N / 2) + (size_t)(n >> 4) * 8 + (n & 7), gated_f(g, u, form));
         }
     }
 }
@@ -1246,12 +1260,12 @@ static void launch_skinny_any(const bf16* x, const bf16* w, TO* out, int M, int 
 
 template <int BM, int BN, int STAGES, int EPI, typename TO, int WM = 2, int WN = 2>
 static int launch_tiled(const bf16* x, const bf16* w, TO* out, float* workspace, int M, int N, int K,
-                        int shares, TailPlan tail, hipStream_t s) {
+                        int shares, TailPlan tail, GateForm form, hipStream_t s) {
     const int tiles_m = (M + BM - 1) / BM, tiles_n = (N + BN - 1) / BN;
     const int tiles = tiles_m * tiles_n;
     if (shares == 1 && tail.shares <= 1) {
         gemm_tiled_kernel<BM, BN, STAGES, EPI, false, TO, WM, WN><<<tiles, 64 * WM * WN, 0, s>>>(
-            x, w, out, nullptr, M, N, K, tiles_m, 0, tiles, 0, g_skew);
+            x, w, out, nullptr, M, N, K, tiles_m, 0, tiles, 0, g_skew, form);
         LC_LAUNCH_CHECK("gemm_tiled");
         return 0;
     }
@@ -1264,22 +1278,22 @@ static int launch_tiled(const bf16* x, const bf16* w, TO* out, float* workspace,
         LC_CHECK(shares == 1 && tail.rest > 0 && tail.rest < tiles, "gemm_bf16: bad tail for tile %dx%d", BM, BN);
         const int whole = tiles - tail.rest;
         gemm_tiled_kernel<BM, BN, STAGES, EPI, false, TO><<<whole, 256, 0, s>>>(
-            x, w, out, nullptr, M, N, K, tiles_m, 0, whole, 0, g_skew);
+            x, w, out, nullptr, M, N, K, tiles_m, 0, whole, 0, g_skew, form);
         LC_LAUNCH_CHECK("gemm_tiled");
         gemm_tiled_kernel<BM, BN, STAGES, 0, true, TO><<<dim3(tail.rest, tail.shares), 256, 0, s>>>(
-            x, w, out, workspace, M, N, K, tiles_m, whole, tail.rest, 1, g_skew);
+            x, w, out, workspace, M, N, K, tiles_m, whole, tail.rest, 1, g_skew, form);
         LC_LAUNCH_CHECK("gemm_tiled");
         tail_reduce_kernel<EPI, TO><<<dim3(tail.rest, (BM * BN + 2047) / 2048), 256, 0, s>>>(
-            workspace, out, M, N, BM, BN, tiles_m, whole, tail.rest, tail.shares);
+            workspace, out, M, N, BM, BN, tiles_m, whole, tail.rest, tail.shares, form);
         LC_LAUNCH_CHECK("tail_reduce");
         return 0;
     } else {
         LC_CHECK(tail.shares <= 1, "gemm_bf16: tile %dx%d has no tail", BM, BN);
         gemm_tiled_kernel<BM, BN, STAGES, 0, true, TO><<<dim3(tiles, shares), 256, 0, s>>>(
-            x, w, out, workspace, M, N, K, tiles_m, 0, tiles, 0, g_skew);
+            x, w, out, workspace, M, N, K, tiles_m, 0, tiles, 0, g_skew, form);
         LC_LAUNCH_CHECK("gemm_tiled");
         const size_t work = EPI ? (size_t)M * N / 2 : (size_t)M * N;
-        splitk_reduce_kernel<EPI, TO><<<(int)((work + 255) / 256), 256, 0, s>>>(workspace, out, M, N, shares);
+        splitk_reduce_kernel<EPI, TO><<<(int)((work + 255) / 256), 256, 0, s>>>(workspace, out, M, N, shares, form);
         LC_LAUNCH_CHECK("splitk_reduce");
         return 0;
     }
@@ -1288,9 +1302,11 @@ static int launch_tiled(const bf16* x, const bf16* w, TO* out, float* workspace,
 
 template <int EPI, typename TO>
 static int launch_bf16(const bf16* x, const bf16* w, TO* out, float* workspace, int M, int N, int K,
-                       hipStream_t s) {
+                       GateForm form, hipStream_t s) {
     if (M <= 16 && g_force_tile == TILE_AUTO) {
-        launch_skinny_any<EPI, false, TO>(x, w, out, M, N, K, SkinnyFuse{}, s);
+        SkinnyFuse fuse{};
+        fuse.form = form;
+        launch_skinny_any<EPI, false, TO>(x, w, out, M, N, K, fuse, s);
         LC_LAUNCH_CHECK("gemm_skinny");
         return 0;
     }
@@ -1298,19 +1314,19 @@ static int launch_bf16(const bf16* x, const bf16* w, TO* out, float* workspace, 
     const int tile = pick_tile(M, N, K);
     const TailPlan tail = tail_plan(tile, M, N, K);
     switch (tile) {
-    case TILE_64x128:  return launch_tiled<64, 128, 3, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_128x128: return launch_tiled<128, 128, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_256x128: return launch_tiled<256, 128, 3, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_256x192: return launch_tiled<256, 192, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_192x128: return launch_tiled<192, 128, 3, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_192x256: return launch_tiled<192, 256, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_64x64:   return launch_tiled<64, 64, 3, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_64x96:   return launch_tiled<64, 96, 6, EPI, TO, 2, 1>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_192x320: return launch_tiled<192, 320, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_64x224:  return launch_tiled<64, 224, 4, EPI, TO, 2, 1>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_64x128_ONE: return launch_tiled<64, 128, 5, EPI, TO, 2, 1>(x, w, out, workspace, M, N, K, shares, tail, s);
-    case TILE_64x160:  return launch_tiled<64, 160, 4, EPI, TO, 2, 1>(x, w, out, workspace, M, N, K, shares, tail, s);
-    default:           return launch_tiled<256, 256, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, s);
+    case TILE_64x128:  return launch_tiled<64, 128, 3, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_128x128: return launch_tiled<128, 128, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_256x128: return launch_tiled<256, 128, 3, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_256x192: return launch_tiled<256, 192, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_192x128: return launch_tiled<192, 128, 3, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_192x256: return launch_tiled<192, 256, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_64x64:   return launch_tiled<64, 64, 3, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_64x96:   return launch_tiled<64, 96, 6, EPI, TO, 2, 1>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_192x320: return launch_tiled<192, 320, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_64x224:  return launch_tiled<64, 224, 4, EPI, TO, 2, 1>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_64x128_ONE: return launch_tiled<64, 128, 5, EPI, TO, 2, 1>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    case TILE_64x160:  return launch_tiled<64, 160, 4, EPI, TO, 2, 1>(x, w, out, workspace, M, N, K, shares, tail, form, s);
+    default:           return launch_tiled<256, 256, 2, EPI, TO>(x, w, out, workspace, M, N, K, shares, tail, form, s);
     }
 }
 
@@ -1360,28 +1376,47 @@ LC_API long long lc_gemm_bf16_workspace(int M, int N, int K) {
     return workspace_words(M, N, K);
 }
 
-// epilogue 0: out[M, N] = x . w^T.  epilogue 1 (SwiGLU): the rows of w come in blocks of 16,
-// 8 gate rows followed by their 8 up rows; out[M, N / 2] = silu(gate) * up.
-// workspace: lc_gemm_bf16_workspace(M, N, K) float32 words (may be null when that is 0).
-LC_API int lc_gemm_bf16(const void* x, const void* w, void* out, int out_dt, int M, int N, int K,
-                        int epilogue, float* workspace, hipStream_t stream) {
+static int check_product(const void* x, const void* w, const void* out, const float* workspace, int M, int N, int K) {
     LC_CHECK(lc_gemm_bf16_supported(M, N, K), "gemm_bf16: sizes M=%d N=%d K=%d are not supported "
              "(K must be a multiple of %d)", M, N, K, SK_KBLOCK);
     LC_CHECK(x && w && out, "gemm_bf16: null pointer");
     LC_CHECK(((uintptr_t)x % 16 == 0) && ((uintptr_t)w % 16 == 0), "gemm_bf16: operands must be 16-byte aligned");
     LC_CHECK((uintptr_t)out % 8 == 0 && (uintptr_t)workspace % 8 == 0, "gemm_bf16: out and workspace must be 8-byte aligned");
-    LC_CHECK(epilogue == 0 || (epilogue == 1 && N % 16 == 0),
-             "gemm_bf16: the SwiGLU epilogue needs N (%d) to be a multiple of 16", N);
-    const bf16* xb = (const bf16*)x;
-    const bf16* wb = (const bf16*)w;
+    return 0;
+}
+
+static int gated_product(const void* x, const void* w, void* out, int out_dt, int M, int N, int K, GateForm form,
+                         float* workspace, hipStream_t stream) {
+    LC_CHECK(N % 16 == 0, "gemm_bf16: the gated epilogue needs N (%d) to be a multiple of 16", N);
     if (out_dt == DT_BF16)
-        return epilogue ? launch_bf16<1, bf16>(xb, wb, (bf16*)out, workspace, M, N, K, stream)
-                        : launch_bf16<0, bf16>(xb, wb, (bf16*)out, workspace, M, N, K, stream);
+        return launch_bf16<1, bf16>((const bf16*)x, (const bf16*)w, (bf16*)out, workspace, M, N, K, form, stream);
     if (out_dt == DT_F32)
-        return epilogue ? launch_bf16<1, float>(xb, wb, (float*)out, workspace, M, N, K, stream)
-                        : launch_bf16<0, float>(xb, wb, (float*)out, workspace, M, N, K, stream);
+        return launch_bf16<1, float>((const bf16*)x, (const bf16*)w, (float*)out, workspace, M, N, K, form, stream);
     LC_CHECK(false, "gemm_bf16: unknown output dtype %d", out_dt);
     return 0;
+}
+
+// epilogue 0: out[M, N] = x . w^T.  epilogue 1 (SwiGLU): the rows of w come in blocks of 16,
+// 8 gate rows followed by their 8 up rows; out[M, N / 2] = silu(gate) * up.
+// workspace: lc_gemm_bf16_workspace(M, N, K) float32 words (may be null when that is 0).
+LC_API int lc_gemm_bf16(const void* x, const void* w, void* out, int out_dt, int M, int N, int K,
+                        int epilogue, float* workspace, hipStream_t stream) {
+    if (int bad = check_product(x, w, out, workspace, M, N, K)) return bad;
+    LC_CHECK(epilogue == 0 || epilogue == 1, "gemm_bf16: unknown epilogue %d", epilogue);
+    if (epilogue) return gated_product(x, w, out, out_dt, M, N, K, kSilu, workspace, stream);
+    const bf16* xb = (const bf16*)x;
+    const bf16* wb = (const bf16*)w;
+    if (out_dt == DT_BF16) return launch_bf16<0, bf16>(xb, wb, (bf16*)out, workspace, M, N, K, kSilu, stream);
+    if (out_dt == DT_F32) return launch_bf16<0, float>(xb, wb, (float*)out, workspace, M, N, K, kSilu, stream);
+    LC_CHECK(false, "gemm_bf16: unknown output dtype %d", out_dt);
+    return 0;
+}
+
+// Epilogue 1 with another gate: g' sigmoid(slope g') (u' + shift), g' = min(g, limit), u' = u inside -limit .. limit.
+LC_API int lc_gemm_bf16_gated(const void* x, const void* w, void* out, int out_dt, int M, int N, int K, float limit,
+                              float slope, float shift, float* workspace, hipStream_t stream) {
+    if (int bad = check_product(x, w, out, workspace, M, N, K)) return bad;
+    return gated_product(x, w, out, out_dt, M, N, K, GateForm{limit, slope, shift}, workspace, stream);
 }
 
 // ------------------------------------------------------------------- norms folded into products
@@ -1447,8 +1482,9 @@ LC_API int lc_gemm_bf16_residual_pieces(int M, int N, int K) {
 
 // resid [M, N] += x [M, K] . w [N, K]^T (float32, in place); next_x [M, N] = bf16(resid * next_w);
 // next_pieces [lc_gemm_bf16_residual_pieces(M, N, K)][stride]: sums of squares of the new rows.
+// bias [N] or null: added to every row of the product.
 LC_API int lc_gemm_bf16_residual(const void* x, const void* w, float* resid, const float* next_w,
-                                 void* next_x, float* next_pieces, int M, int N, int K,
+                                 void* next_x, float* next_pieces, const float* bias, int M, int N, int K,
                                  hipStream_t stream) {
     LC_CHECK(lc_gemm_bf16_residual_pieces(M, N, K) > 0,
              "gemm_bf16_residual: sizes M=%d N=%d K=%d are not supported", M, N, K);
@@ -1459,6 +1495,7 @@ LC_API int lc_gemm_bf16_residual(const void* x, const void* w, float* resid, con
     fuse.next_w = next_w;
     fuse.next_x = (bf16*)next_x;
     fuse.next_partials = next_pieces;
+    fuse.resid_bias = bias;
     fuse.stride = lc_gemm_bf16_piece_stride(M);
     launch_skinny_any<2, false, float>((const bf16*)x, (const bf16*)w, (float*)nullptr, M, N, K, fuse, stream);
     LC_LAUNCH_CHECK("gemm_skinny");
@@ -1471,10 +1508,10 @@ LC_API int lc_gemm_bf16_scaled_rows_supported(int M, int N, int K) {
 }
 
 // out = (x . w^T) with row m scaled by rsqrt(sum_p pieces[p][m] / K + eps) before the epilogue
-// (0: plain, bfloat16 [M, N]; 1: SwiGLU as in lc_gemm_bf16, bfloat16 [M, N / 2]).
+// (0: plain, bfloat16 [M, N]; 1: gated as in lc_gemm_bf16_gated, bfloat16 [M, N / 2]).
 LC_API int lc_gemm_bf16_scaled_rows(const void* x, const void* w, void* out, int M, int N, int K,
-                                    int epilogue, const float* pieces, int count, float eps,
-                                    hipStream_t stream) {
+                                    int epilogue, float limit, float slope, float shift, const float* pieces,
+                                    int count, float eps, hipStream_t stream) {
     LC_CHECK(lc_gemm_bf16_scaled_rows_supported(M, N, K),
              "gemm_bf16_scaled_rows: sizes M=%d N=%d K=%d are not supported", M, N, K);
     LC_CHECK(count >= 1 && count <= SK_MAX_PIECES, "gemm_bf16_scaled_rows: %d pieces (at most %d)", count, SK_MAX_PIECES);
@@ -1486,6 +1523,7 @@ LC_API int lc_gemm_bf16_scaled_rows(const void* x, const void* w, void* out, int
     fuse.scale_partials = pieces;
     fuse.scale_count = count;
     fuse.scale_eps = eps;
+    fuse.form = GateForm{limit, slope, shift};
     fuse.stride = lc_gemm_bf16_piece_stride(M);
     if (epilogue) launch_skinny_any<1, true, bf16>((const bf16*)x, (const bf16*)w, (bf16*)out, M, N, K, fuse, stream);
     else launch_skinny_any<0, true, bf16>((const bf16*)x, (const bf16*)w, (bf16*)out, M, N, K, fuse, stream);
@@ -1519,15 +1557,15 @@ LC_API int lc_gemm_bf16_partials(const void* x, const void* w, float* partials, 
     if (pick_tile(M, N, K, true) == TILE_64x64) {
         const int tiles_m = (M + 63) / 64, tiles = tiles_m * ((N + 63) / 64);
         gemm_tiled_kernel<64, 64, 3, 0, true, float><<<dim3(tiles, shares), 256, 0, stream>>>(
-            xb, wb, nullptr, partials, M, N, K, tiles_m, 0, tiles, 0, g_skew);
+            xb, wb, nullptr, partials, M, N, K, tiles_m, 0, tiles, 0, g_skew, kSilu);
     } else if (pick_tile(M, N, K, true) == TILE_64x128) {
         const int tiles_m = (M + 63) / 64, tiles = tiles_m * ((N + 127) / 128);
         gemm_tiled_kernel<64, 128, 3, 0, true, float><<<dim3(tiles, shares), 256, 0, stream>>>(
-            xb, wb, nullptr, partials, M, N, K, tiles_m, 0, tiles, 0, g_skew);
+            xb, wb, nullptr, partials, M, N, K, tiles_m, 0, tiles, 0, g_skew, kSilu);
     } else {
         const int tiles_m = (M + 127) / 128, tiles = tiles_m * ((N + 127) / 128);
         gemm_tiled_kernel<128, 128, 2, 0, true, float><<<dim3(tiles, shares), 256, 0, stream>>>(
-            xb, wb, nullptr, partials, M, N, K, tiles_m, 0, tiles, 0, g_skew);
+            xb, wb, nullptr, partials, M, N, K, tiles_m, 0, tiles, 0, g_skew, kSilu);
     }
     LC_LAUNCH_CHECK("gemm_tiled");
     return 0;
@@ -1542,8 +1580,8 @@ LC_API int lc_gemm_bf16_sum_shares(const float* partials, void* out, int dt, int
     if (M == 0) return 0;
     const size_t work = (size_t)M * N;
     const int blocks = (int)((work + 255) / 256 < 65535 * 16 ? (work + 255) / 256 : 65535 * 16);
-    if (dt == DT_BF16) splitk_reduce_kernel<0, bf16><<<blocks, 256, 0, stream>>>(partials, (bf16*)out, M, N, shares);
-    else if (dt == DT_F32) splitk_reduce_kernel<0, float><<<blocks, 256, 0, stream>>>(partials, (float*)out, M, N, shares);
+    if (dt == DT_BF16) splitk_reduce_kernel<0, bf16><<<blocks, 256, 0, stream>>>(partials, (bf16*)out, M, N, shares, kSilu);
+    else if (dt == DT_F32) splitk_reduce_kernel<0, float><<<blocks, 256, 0, stream>>>(partials, (float*)out, M, N, shares, kSilu);
     else LC_CHECK(false, "gemm_bf16_sum_shares: unknown dtype %d", dt);
     LC_LAUNCH_CHECK("splitk_reduce");
     return 0;

@@ -5,7 +5,7 @@
 //   with a stream   v = h + d, where d is the branch output, itself layer-normed first if it
 //                   brings weights of its own; h becomes v where asked
 //   position vector entry 2i: sin(p f_i), entry 2i + 1: cos(p f_i)
-//   gated           act(gate) * up, act = silu or gelu (tanh form)
+//   gated           act(gate) * up, act = silu or gelu (tanh form); or both clamped, a steeper sigmoid, up shifted
 //   heads in slots  q, k heads divided by their root mean square over their own entries, times a
 //                   weight, q also times a factor per head; q, k, v written as heads of `slot`
 //                   entries with zeros behind theirs (k, v into the paged cache)
@@ -162,11 +162,18 @@ __global__ void embedding_sinusoid_kernel(const int* __restrict__ ids, const int
 }
 
 template <typename T>
-__global__ void gated_activation_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, int kind, size_t total) {
+__global__ void gated_activation_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, int kind, float limit,
+                                        float slope, float shift, size_t total) {
     for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
          idx += (size_t)gridDim.x * blockDim.x) {
         const size_t t = idx / I, i = idx % I;
-        const float g = to_f32(gu[t * 2 * I + i]), u = to_f32(gu[t * 2 * I + I + i]);
+        float g = to_f32(gu[t * 2 * I + i]), u = to_f32(gu[t * 2 * I + I + i]);
+        if (kind == 2) {
+            g = fminf(g, limit);
+            u = fminf(fmaxf(u, -limit), limit);
+            out[idx] = from_f32<T>(g * sigmoid(slope * g) * (u + shift));
+            continue;
+        }
         out[idx] = from_f32<T>((kind == 0 ? silu(g) : activate(g, ACT_GELU_TANH)) * u);
     }
 }
@@ -300,16 +307,20 @@ LC_API int lc_embedding_sinusoid(const int* ids, const int* positions, const voi
     return 0;
 }
 
-// gu [T, 2 I] -> out [T, I]; kind 0: silu, 1: gelu (tanh form)
-LC_API int lc_gated_activation(const void* gu, void* out, int dt, int T, int I, int kind, hipStream_t stream) {
-    LC_CHECK(T >= 0 && I > 0 && (kind == 0 || kind == 1), "gated_activation: bad arguments");
+// gu [T, 2 I] -> out [T, I]; kind 0: silu, 1: gelu (tanh form), 2: g' sigmoid(slope g') (u' + shift) with
+// g' = min(g, limit) and u' = u inside -limit .. limit
+LC_API int lc_gated_activation(const void* gu, void* out, int dt, int T, int I, int kind, float limit, float slope,
+                               float shift, hipStream_t stream) {
+    LC_CHECK(T >= 0 && I > 0 && kind >= 0 && kind <= 2, "gated_activation: bad arguments");
     if (T == 0) return 0;
     LC_CHECK(gu && out, "gated_activation: null pointer");
     const size_t total = (size_t)T * I;
     if (dt == DT_F32)
-        gated_activation_kernel<float><<<blocks_for(total), 256, 0, stream>>>((const float*)gu, (float*)out, I, kind, total);
+        gated_activation_kernel<float><<<blocks_for(total), 256, 0, stream>>>((const float*)gu, (float*)out, I, kind, limit,
+                                                                            slope, shift, total);
     else if (dt == DT_BF16)
-        gated_activation_kernel<bf16><<<blocks_for(total), 256, 0, stream>>>((const bf16*)gu, (bf16*)out, I, kind, total);
+        gated_activation_kernel<bf16><<<blocks_for(total), 256, 0, stream>>>((const bf16*)gu, (bf16*)out, I, kind, limit,
+                                                                           slope, shift, total);
     else
         LC_CHECK(false, "gated_activation: unknown dtype %d", dt);
     LC_LAUNCH_CHECK("gated_activation");

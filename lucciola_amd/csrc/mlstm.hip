@@ -1,0 +1,219 @@
+// The matrix memory of the xLSTM (mLSTM) around the framework's recurrence kernel.  Per head, with the state S
+// [key, value], the normaliser n [key] and the reference point m (float32, all zero at a sequence's start):
+//   i = cap tanh((x_i + b_i) / cap),   f = logsigmoid(cap tanh((x_f + b_f) / cap))       (logarithms of the gates)
+//   m' = max(f + m, i);   S <- e^(f + m - m') S + e^(i - m') k v^T;   n <- e^(f + m - m') n + e^(i - m') k
+//   o = S^T q / (max(|n . q|, e^(-m')) + floor)
+// The normaliser is one more value channel, whose value is 1 in every token: with it beside the others the
+// recurrence is S <- diag(decay) S + write v^T, o = S^T read without a removal term, with decay = e^(f + m - m') in
+// every key channel, write = e^(i - m') k, read = q_scale q.  This file makes those inputs from a step's float32
+// projections: the reference points, which tie a token to the one before it, by one wave per request and head that
+// walks the request's tokens; the vectors by a thread an entry.  A step of lone tokens does both in one kernel.
+// Behind the scan the read-out divides by the normaliser, takes each head by its root mean square, multiplies by a
+// weight and sigmoid(gate) and rounds to the activation type; everything before that rounding is float32.
+#include "common.h"
+
+#include "activations.h"
+
+namespace lc {
+
+// What the token's gates make of the reference point before it.
+struct MemoryGates {
+    float keep_log, write_log;
+};
+__device__ __forceinline__ MemoryGates memory_gates(float x_i, float b_i, float x_f, float b_f, float cap) {
+    const float z = cap * tanhf((x_f + b_f) / cap);
+    return {fminf(z, 0.f) - log1pf(expf(-fabsf(z))), cap * tanhf((x_i + b_i) / cap)};
+}
+__device__ __forceinline__ float next_reference(const MemoryGates& g, float m) { return fmaxf(g.keep_log + m, g.write_log); }
+__device__ __forceinline__ float keep_factor(const MemoryGates& g, float before, float after) {
+    return expf(g.keep_log + before - after);
+}
+__device__ __forceinline__ float write_factor(const MemoryGates& g, float after) { return expf(g.write_log - after); }
+
+__device__ __forceinline__ float from_lane(float v, int lane) {
+    return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane));
+}
+
+// grid (heads, requests), one wave.  proj [T, cols] with x_i at columns i_col + head and x_f at f_col + head;
+// factors [3, T, heads]: keep, write and e^(-m') of every token; reference [slots, heads].
+// 64 tokens at a time: their gates side by side, then the chain of maxima, one add and one max a token, in order, so
+// that a token's numbers have the same bits however its request is cut into steps.
+__global__ __launch_bounds__(kWave) void mlstm_gates_kernel(
+    const float* __restrict__ proj, int cols, int i_col, int f_col, const float* __restrict__ i_bias,
+    const float* __restrict__ f_bias, float cap, float* __restrict__ reference, const int* __restrict__ q_offsets,
+    const int* __restrict__ slot_ids, int T, int heads, float* __restrict__ factors) {
+    const int head = blockIdx.x, req = blockIdx.y, lane = threadIdx.x;
+    const int first = q_offsets[req], last = q_offsets[req + 1];
+    float* home = reference + (size_t)slot_ids[req] * heads + head;
+    const size_t plane = (size_t)T * heads;
+    const float b_i = i_bias[head], b_f = f_bias[head];
+    float m = *home;
+    auto fetch = [&](int t0, float& x_i, float& x_f) {
+        const int t = min(t0 + lane, last - 1);
+        x_i = proj[(size_t)t * cols + i_col + head];
+        x_f = proj[(size_t)t * cols + f_col + head];
+    };
+    float x_i = 0.f, x_f = 0.f;
+    if (first < last) fetch(first, x_i, x_f);
+    for (int t0 = first; t0 < last; t0 += kWave) {
+        const int count = min(kWave, last - t0);
+        MemoryGates g = memory_gates(x_i, b_i, x_f, b_f, cap);
+        if (t0 + kWave < last) fetch(t0 + kWave, x_i, x_f);     // on their way during the chain
+        if (lane >= count) g = {0.f, -INFINITY};                // behind the request's end: nothing moves
+        const float entry = m;
+        float after = m;
+#pragma unroll
+        for (int k = 0; k < kWave; ++k) {
+            m = fmaxf(from_lane(g.keep_log, k) + m, from_lane(g.write_log, k));
+            after = lane == k ? m : after;
+        }
+        float before = __shfl_up(after, 1, kWave);
+        if (lane == 0) before = entry;
+        if (lane < count) {
+            const size_t at = (size_t)(t0 + lane) * heads + head;
+            factors[at] = keep_factor(g, before, after);
+            factors[plane + at] = write_factor(g, after);
+            factors[2 * plane + at] = expf(-after);
+        }
+    }
+    if (lane == 0 && first < last) *home = m;
+}
+
+// A thread per entry.  proj [T, cols]: q | k (heads x dk each) | v (heads x dv) | ...; coef [3, T, heads dk]: decay,
+// write, read; v_out [T, heads (dv + 1)], a 1 behind every head's values.
+__global__ void mlstm_prepare_kernel(const float* __restrict__ proj, int cols, int T, int heads, int dk, int dv,
+                                     float q_scale, const float* __restrict__ factors, float* __restrict__ coef,
+                                     float* __restrict__ v_out) {
+    const int nk = heads * dk, nv = heads * (dv + 1);
+    const size_t plane = (size_t)T * nk, total = (size_t)T * (nk + nv);
+    for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
+         idx += (size_t)gridDim.x * blockDim.x) {
+        const int t = (int)(idx / (nk + nv)), c = (int)(idx % (nk + nv));
+        const float* row = proj + (size_t)t * cols;
+        if (c < nk) {
+            const size_t at = (size_t)t * nk + c, f = (size_t)t * heads + c / dk;
+            coef[at] = factors[f];
+            coef[plane + at] = factors[(size_t)T * heads + f] * row[nk + c];
+            coef[2 * plane + at] = q_scale * row[c];
+        } else {
+            const int head = (c - nk) / (dv + 1), e = (c - nk) % (dv + 1);
+            v_out[(size_t)t * nv + (c - nk)] = e < dv ? row[2 * nk + head * dv + e] : 1.f;
+        }
+    }
+}
+
+// The two above for a step whose requests bring one token each: grid (requests, heads), a workgroup per token and head.
+__global__ void mlstm_lone_kernel(const float* __restrict__ proj, int cols, int i_col, int f_col,
+                                  const float* __restrict__ i_bias, const float* __restrict__ f_bias, float cap,
+                                  float* __restrict__ reference, const int* __restrict__ q_offsets,
+                                  const int* __restrict__ slot_ids, int T, int heads, int dk, int dv, float q_scale,
+                                  float* __restrict__ factors, float* __restrict__ coef, float* __restrict__ v_out) {
+    const int req = blockIdx.x, head = blockIdx.y, t = q_offsets[req];
+    float* home = reference + (size_t)slot_ids[req] * heads + head;
+    const float* row = proj + (size_t)t * cols;
+    const float m = *home;
+    const MemoryGates g = memory_gates(row[i_col + head], i_bias[head], row[f_col + head], f_bias[head], cap);
+    const float after = next_reference(g, m);
+    const float keep = keep_factor(g, m, after), write = write_factor(g, after);
+    const int nk = heads * dk;
+    const size_t plane = (size_t)T * nk, at0 = (size_t)t * nk + (size_t)head * dk;
+    for (int e = threadIdx.x; e < dk; e += blockDim.x) {
+        coef[at0 + e] = keep;
+        coef[plane + at0 + e] = write * row[nk + head * dk + e];
+        coef[2 * plane + at0 + e] = q_scale * row[head * dk + e];
+    }
+    float* v = v_out + ((size_t)t * heads + head) * (dv + 1);
+    for (int e = threadIdx.x; e <= dv; e += blockDim.x) v[e] = e < dv ? row[2 * nk + head * dv + e] : 1.f;
+    __syncthreads();            // every thread has read the reference point
+    if (threadIdx.x == 0) {
+        *home = after;
+        const size_t f = (size_t)t * heads + head, fp = (size_t)T * heads;
+        factors[f] = keep;
+        factors[fp + f] = write;
+        factors[2 * fp + f] = expf(-after);
+    }
+}
+
+constexpr int READ_WAVES = 4;
+
+// One wave per (token, head).  o [T, heads (dv + 1)]: a head's read-outs, then its normaliser's; bottoms [T, heads]
+// (e^(-m')); gates: columns gate_column .. + heads dv of [T, gate_cols]; weight [heads dv].
+template <typename T>
+__global__ __launch_bounds__(READ_WAVES * kWave) void mlstm_readout_kernel(
+    const float* __restrict__ o, const float* __restrict__ bottoms, float floor_, const float* __restrict__ gates,
+    int gate_cols, int gate_column, const float* __restrict__ weight, float eps, int rows, int heads, int dv,
+    T* __restrict__ out) {
+    const int row = blockIdx.x * READ_WAVES + threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
+    if (row >= rows) return;
+    const int t = row / heads, head = row % heads;
+    const float* mine = o + (size_t)row * (dv + 1);
+    const float inv = 1.f / (fmaxf(fabsf(mine[dv]), bottoms[row]) + floor_);
+    float ss = 0.f;
+    for (int e = lane; e < dv; e += kWave) {
+        const float v = mine[e] * inv;
+        ss = fmaf(v, v, ss);
+    }
+    const float by = inv / sqrtf(wave_sum(ss) / (float)dv + eps);
+    for (int e = lane; e < dv; e += kWave) {
+        const int c = head * dv + e;
+        out[(size_t)t * heads * dv + c] =
+            from_f32<T>(mine[e] * by * weight[c] * sigmoid(gates[(size_t)t * gate_cols + gate_column + c]));
+    }
+}
+
+}  // namespace lc
+
+using namespace lc;
+
+// factors [3, T, heads], coef [3, T, heads dk], v_out [T, heads (dv + 1)].  lone: every request brings one token.
+LC_API int lc_mlstm_prepare(const float* proj, int cols, int i_col, int f_col, const float* i_bias, const float* f_bias,
+                            float cap, float* reference, int slots, const int* q_offsets, const int* slot_ids, int R,
+                            int T, int heads, int dk, int dv, float q_scale, int lone, float* factors, float* coef,
+                            float* v_out, hipStream_t stream) {
+    LC_CHECK(R >= 0 && T >= R && heads > 0 && dk > 0 && dv > 0 && slots >= 0 && cap > 0.f, "mlstm prepare: bad sizes");
+    LC_CHECK(i_col >= 0 && f_col >= 0 && i_col + heads <= cols && f_col + heads <= cols && heads * (2 * dk + dv) <= cols,
+             "mlstm prepare: the columns do not fit the heads");
+    LC_CHECK(!lone || T == R, "mlstm prepare: %d tokens are not lone tokens of %d requests", T, R);
+    if (T == 0 || R == 0) return 0;
+    LC_CHECK(proj && i_bias && f_bias && reference && q_offsets && slot_ids && factors && coef && v_out,
+             "mlstm prepare: null pointer");
+    LC_CHECK(R <= 65535 && heads <= 65535, "mlstm prepare: too many requests or heads for the grid");
+    if (lone) {
+        const int widest = dk > dv + 1 ? dk : dv + 1;
+        const int threads = widest > 128 ? 256 : (widest > 64 ? 128 : 64);
+        mlstm_lone_kernel<<<dim3(R, heads), threads, 0, stream>>>(proj, cols, i_col, f_col, i_bias, f_bias, cap, reference,
+                                                                  q_offsets, slot_ids, T, heads, dk, dv, q_scale, factors,
+                                                                  coef, v_out);
+        LC_LAUNCH_CHECK("mlstm_lone");
+        return 0;
+    }
+    mlstm_gates_kernel<<<dim3(heads, R), kWave, 0, stream>>>(proj, cols, i_col, f_col, i_bias, f_bias, cap, reference,
+                                                             q_offsets, slot_ids, T, heads, factors);
+    LC_LAUNCH_CHECK("mlstm_gates");
+    const size_t total = (size_t)T * heads * (dk + dv + 1);
+    const int blocks = (int)((total + 255) / 256 < 16384 ? (total + 255) / 256 : 16384);
+    mlstm_prepare_kernel<<<blocks, 256, 0, stream>>>(proj, cols, T, heads, dk, dv, q_scale, factors, coef, v_out);
+    LC_LAUNCH_CHECK("mlstm_prepare");
+    return 0;
+}
+
+LC_API int lc_mlstm_readout(const float* o, const float* bottoms, float floor_, const float* gates, int gate_cols,
+                            int gate_column, const float* weight, float eps, int T, int heads, int dv, void* out, int dt,
+                            hipStream_t stream) {
+    LC_CHECK(T >= 0 && heads > 0 && dv > 0 && gate_column >= 0 && gate_column + heads * dv <= gate_cols,
+             "mlstm readout: bad sizes");
+    if (T == 0) return 0;
+    LC_CHECK(o && bottoms && gates && weight && out, "mlstm readout: null pointer");
+    LC_CHECK((long long)T * heads < (1ll << 31), "mlstm readout: too many heads");
+    const int rows = T * heads, blocks = (rows + READ_WAVES - 1) / READ_WAVES;
+    if (dt == DT_F32)
+        mlstm_readout_kernel<float><<<blocks, READ_WAVES * kWave, 0, stream>>>(o, bottoms, floor_, gates, gate_cols, gate_column,
+                                                                               weight, eps, rows, heads, dv, (float*)out);
+    else if (dt == DT_BF16)
+        mlstm_readout_kernel<bf16><<<blocks, READ_WAVES * kWave, 0, stream>>>(o, bottoms, floor_, gates, gate_cols, gate_column,
+                                                                              weight, eps, rows, heads, dv, (bf16*)out);
+    else
+        LC_CHECK(false, "mlstm readout: unknown dtype %d", dt);
+    LC_LAUNCH_CHECK("mlstm_readout");
+    return 0;
+}

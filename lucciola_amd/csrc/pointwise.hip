@@ -59,6 +59,15 @@ __global__ void activation_kernel(T* __restrict__ x, int kind, float a, float b,
     }
 }
 
+// out[t] = x[t] + bias, for every row t
+template <typename T>
+__global__ void bias_add_kernel(const T* __restrict__ x, const float* __restrict__ bias, T* __restrict__ out, int n,
+                                size_t total) {
+    for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
+         idx += (size_t)gridDim.x * blockDim.x)
+        out[idx] = from_f32<T>(to_f32(x[idx]) + bias[idx % n]);
+}
+
 __global__ void scale_kernel(float* __restrict__ x, float factor, size_t total) {
     for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
          idx += (size_t)gridDim.x * blockDim.x)
@@ -245,5 +254,18 @@ LC_API int lc_rms_shift(const float* h, const void* delta, int dt_delta, float* 
     else LC_CHECK(false, "rms_shift: unknown dtypes %d, %d", dt, dt_delta);
 #undef LC_RS
     LC_LAUNCH_CHECK("rms_shift");
+    return 0;
+}
+
+LC_API int lc_bias_add(const void* x, int dt, const float* bias, void* out, int T, int n, hipStream_t stream) {
+    LC_CHECK(T >= 0 && n > 0, "bias_add: bad sizes");
+    if (T == 0) return 0;
+    LC_CHECK(x && bias && out, "bias_add: null pointer");
+    const size_t total = (size_t)T * n;
+    const int blocks = (int)((total + 255) / 256 < 8192 ? (total + 255) / 256 : 8192);
+    if (dt == DT_F32) bias_add_kernel<float><<<blocks, 256, 0, stream>>>((const float*)x, bias, (float*)out, n, total);
+    else if (dt == DT_BF16) bias_add_kernel<bf16><<<blocks, 256, 0, stream>>>((const bf16*)x, bias, (bf16*)out, n, total);
+    else LC_CHECK(false, "bias_add: unknown dtype %d", dt);
+    LC_LAUNCH_CHECK("bias_add");
     return 0;
 }

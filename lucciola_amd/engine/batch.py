@@ -129,6 +129,9 @@ class StepBatch:
     plans: Dict[Any, Plan] = field(default_factory=dict)   # by planner key
     num_wanted: int = 0
     buffer: Optional[torch.Tensor] = None   # the one device buffer all of the above view
+    # what a layer's part leaves, by name, for the same tokens in later layers of this pass through the model (a
+    # layer's values that later layers mix in); empty before and after a pass
+    passing: Dict[str, torch.Tensor] = field(default_factory=dict)
 
 
 class _Packer:

@@ -26,10 +26,11 @@ DT_F32, DT_BF16 = 0, 1
 _ARG = {"p": ctypes.c_void_p, "i": ctypes.c_int, "f": ctypes.c_float, "q": ctypes.c_longlong}
 _SIGNATURES = {
     "lc_embedding": "ppipiiifp",
-    "lc_rmsnorm": "ppppfpiiiipiip",
+    "lc_rmsnorm": "ppppfpiiiipiipp",
     "lc_rmsnorm_act": "pqpfpiiip",
     "lc_gemm_generic": "pipipiiiipp",
     "lc_gemm_bf16": "pppiiiiipp",
+    "lc_gemm_bf16_gated": "pppiiiifffpp",
     "lc_gemm_bf16_supported": "iii",
     "lc_gemm_bf16_kblock": "",
     "lc_gemm_bf16_force_tile": "i",
@@ -44,8 +45,8 @@ _SIGNATURES = {
     "lc_gemm_bf16_shares": "iii",
     "lc_gemm_bf16_tile": "iiii",
     "lc_gemm_bf16_partials": "pppiiip",
-    "lc_gemm_bf16_residual": "ppppppiiip",
-    "lc_gemm_bf16_scaled_rows": "pppiiiipifp",
+    "lc_gemm_bf16_residual": "pppppppiiip",
+    "lc_gemm_bf16_scaled_rows": "pppiiiifffpifp",
     "lc_gemm_bf16_scaled_rows_supported": "iii",
     "lc_qk_norm_rope_write": "piiiiippfppipppiip",
     "lc_attention_generic": "pipppipppiiiiiifipp",
@@ -93,7 +94,7 @@ _SIGNATURES = {
     "lc_moe_combine": "pppiiipip",
     "lc_layer_norm": "ppifppfpppfpiiiiip",
     "lc_embedding_sinusoid": "pppippiiifp",
-    "lc_gated_activation": "ppiiiip",
+    "lc_gated_activation": "ppiiiifffp",
     "lc_head_norm_write": "piiiiiiippfpppppiip",
     "lc_general_delta_prepare": "piiiipppffppp",
     "lc_gated_delta_prepare": "piiiiiippippfpppppp",
@@ -113,6 +114,10 @@ _SIGNATURES = {
     "lc_state_space_prepare": "piiiiii" + "ppi" + "ppp" + "ppp" + "pp" + "p",
     "lc_state_space_readout": "pppiipiipifipip",
     "lc_scaled_sum": "pifpifpqp",
+    "lc_bias_add": "pippiip",
+    "lc_attention_rows": "piiiiiii" + "pppf" + "piip" + "pfp" + "pppipi" + "p",
+    "lc_mlstm_prepare": "piiippf" + "pippi" + "iiiifi" + "ppp" + "p",
+    "lc_mlstm_readout": "ppfpiipfiiipip",
 }
 
 
@@ -274,6 +279,19 @@ class PendingProduct:
 
 
 @dataclass
+class BiasedBranch:
+    """A branch's output ``branch`` (a tensor [T, n] or a PendingProduct) that still lacks its ``bias`` [n] float32:
+    :func:`rmsnorm` takes it as the stream's pending addition and adds both in float32; anyone else gets the
+    sum from ``value()``."""
+
+    branch: object
+    bias: torch.Tensor
+
+    def value(self) -> torch.Tensor:
+        return bias_add(value(self.branch), self.bias)
+
+
+@dataclass
 class ScaledRows:
     """The normed residual stream short of each row's factor: ``x`` = bf16(h * weight) [T, n];
     ``pieces`` [count, T rounded up to a power of two] float32 hold pieces of the rows' sums of
@@ -314,13 +332,13 @@ class ProductShares:
 
 def value(t):
     """The tensor that ``t`` stands for (``t`` itself if it is one)."""
-    return t.value() if isinstance(t, (PendingProduct, ScaledRows, ProductShares, NormedBranch)) else t
+    return t.value() if isinstance(t, (PendingProduct, ScaledRows, ProductShares, NormedBranch, BiasedBranch)) else t
 
 
 def rmsnorm(h: torch.Tensor, delta, weight: torch.Tensor, eps: float,
             out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None, scaled: bool = False):
     """RMSNorm of the float32 residual stream ``h`` [T, n], with the pending branch output
-    ``delta`` [T, n] (a tensor or a PendingProduct) added first.
+    ``delta`` [T, n] (a tensor, a PendingProduct or a BiasedBranch) added first.
 
     Without ``rows``: ``h += delta`` in place and every row is normed.  With ``rows`` (int32
     [R]): only those rows are normed (``h`` stays as it is) and the result is [R, n].
@@ -333,6 +351,12 @@ def rmsnorm(h: torch.Tensor, delta, weight: torch.Tensor, eps: float,
         raise KernelError(f"rmsnorm: weight has {weight.shape[0]} entries for rows of {n}")
     scaled = (scaled and rows is None and out_dtype == torch.bfloat16 and T > 0
               and bool(library().lc_gemm_bf16_scaled_rows_supported(T, 16, n)))
+    bias = None
+    if isinstance(delta, BiasedBranch):
+        delta, bias = delta.branch, delta.bias
+        _need(bias, "rmsnorm branch bias", torch.float32, 1)
+        if bias.shape[0] != n:
+            raise KernelError(f"rmsnorm: the branch's bias has {bias.shape[0]} entries for rows of {n}")
     if isinstance(delta, PendingProduct):
         M, K = delta.x.shape
         pieces = (library().lc_gemm_bf16_residual_pieces(M, n, K)
@@ -342,7 +366,7 @@ def rmsnorm(h: torch.Tensor, delta, weight: torch.Tensor, eps: float,
             parts = torch.empty((pieces, library().lc_gemm_bf16_piece_stride(T)), dtype=torch.float32,
                                 device=h.device)
             _call("lc_gemm_bf16_residual", _ptr(delta.x), _ptr(delta.w), _ptr(h), _ptr(weight),
-                  _ptr(xg), _ptr(parts), _c_int(M), _c_int(n), _c_int(K), _stream())
+                  _ptr(xg), _ptr(parts), _ptr(bias), _c_int(M), _c_int(n), _c_int(K), _stream())
             return ScaledRows(xg, parts, pieces, float(eps), h, weight)
         shares = library().lc_gemm_bf16_shares(M, n, K) if (delta.w.shape[0] == n and M == T) else 0
         if shares:
@@ -369,7 +393,7 @@ def rmsnorm(h: torch.Tensor, delta, weight: torch.Tensor, eps: float,
     _call("lc_rmsnorm", _ptr(h), _ptr(delta), _ptr(rows), _ptr(weight), _c_float(eps), _ptr(out),
           _c_int(_dt(out)), _c_int(R), _c_int(n),
           _c_int(1 if (rows is None and delta is not None) else 0), _ptr(parts), _c_int(shares),
-          _c_int(T), _stream())
+          _c_int(T), _ptr(bias), _stream())
     return ScaledRows(out, parts, 1, float(eps), h, weight) if scaled else out
 
 
@@ -395,7 +419,20 @@ def rmsnorm_act(x: torch.Tensor, weight: torch.Tensor, eps: float, column: Optio
 
 
 # ------------------------------------------------------------------------------ products
-def _scaled_product(x: "ScaledRows", w: torch.Tensor, epilogue: int) -> Optional[torch.Tensor]:
+@dataclass(frozen=True)
+class GateForm:
+    """What a gated feed-forward makes of a gate entry g and an up entry u: with g' = min(g, limit) and u' = u held
+    inside -limit .. limit, g' sigmoid(slope g') (u' + shift).  The defaults are silu(g) u."""
+
+    limit: float = float("inf")
+    slope: float = 1.0
+    shift: float = 0.0
+
+
+SILU_GATE = GateForm()
+
+
+def _scaled_product(x: "ScaledRows", w: torch.Tensor, epilogue: int, form: GateForm = SILU_GATE) -> Optional[torch.Tensor]:
     """``x`` with its rows' factors times ``w`` transposed in one kernel, or None if there is
     no such kernel for these operands."""
     M, K = x.x.shape
@@ -405,7 +442,7 @@ def _scaled_product(x: "ScaledRows", w: torch.Tensor, epilogue: int) -> Optional
         return None
     out = torch.empty((M, N // 2 if epilogue else N), dtype=torch.bfloat16, device=w.device)
     _call("lc_gemm_bf16_scaled_rows", _ptr(x.x), _ptr(w), _ptr(out), _c_int(M), _c_int(N),
-          _c_int(K), _c_int(epilogue), _ptr(x.pieces), _c_int(x.count), _c_float(x.eps), _stream())
+          _c_int(K), _c_int(epilogue), _c_float(form.limit), _c_float(form.slope), _c_float(form.shift), _ptr(x.pieces), _c_int(x.count), _c_float(x.eps), _stream())
     return out
 
 
@@ -470,12 +507,12 @@ def gemm_swiglu_supported(x_dtype, w: torch.Tensor, K: int) -> bool:
             and _fast_gemm_ok(64, w.shape[0], K))
 
 
-def gemm_swiglu(x: torch.Tensor, w_interleaved: torch.Tensor) -> torch.Tensor:
-    """``silu(x . gate^T) * (x . up^T)`` in one kernel, with gate and up interleaved by
-    :func:`interleave_gate_up`; bfloat16 only.  [M, K] x [2 I, K] -> [M, I].  ``x`` may be
+def gemm_swiglu(x: torch.Tensor, w_interleaved: torch.Tensor, form: GateForm = SILU_GATE) -> torch.Tensor:
+    """``silu(x . gate^T) * (x . up^T)`` (or what ``form`` makes of the two) in one kernel, with gate and up
+    interleaved by :func:`interleave_gate_up`; bfloat16 only.  [M, K] x [2 I, K] -> [M, I].  ``x`` may be
     ScaledRows."""
     if isinstance(x, ScaledRows):
-        out = _scaled_product(x, w_interleaved, 1) if w_interleaved.shape[0] % 16 == 0 else None
+        out = _scaled_product(x, w_interleaved, 1, form) if w_interleaved.shape[0] % 16 == 0 else None
         if out is not None:
             return out
         x = x.value()
@@ -486,7 +523,10 @@ def gemm_swiglu(x: torch.Tensor, w_interleaved: torch.Tensor) -> torch.Tensor:
     if K != K2 or N % 16:
         raise KernelError(f"gemm_swiglu: x is [{M}, {K}], w is [{N}, {K2}] (rows must come in 16s)")
     out = torch.empty((M, N // 2), dtype=torch.bfloat16, device=x.device)
-    if M:
+    if M and form is not SILU_GATE:
+        _call("lc_gemm_bf16_gated", _ptr(x), _ptr(w_interleaved), _ptr(out), DT_BF16, M, N, K, float(form.limit),
+              float(form.slope), float(form.shift), _ptr(_gemm_workspace(M, N, K, x.device)), _stream())
+    elif M:
         _call("lc_gemm_bf16", _ptr(x), _ptr(w_interleaved), _ptr(out), DT_BF16, M, N, K, 1,
               _ptr(_gemm_workspace(M, N, K, x.device)), _stream())
     return out
@@ -1474,15 +1514,17 @@ def embedding_sinusoid(ids: torch.Tensor, table: torch.Tensor, positions: torch.
 GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
 
 
-def gated_activation(gu: torch.Tensor, kind: str) -> torch.Tensor:
-    """``gu`` [T, 2 I] (gate columns, then up columns) -> act(gate) * up, [T, I]; float32 arithmetic."""
+def gated_activation(gu: torch.Tensor, kind: str, form: Optional[GateForm] = None) -> torch.Tensor:
+    """``gu`` [T, 2 I] (gate columns, then up columns) -> act(gate) * up, [T, I]; float32 arithmetic.  With
+    ``form`` (and ``kind`` "silu"): what it makes of the two."""
     _need(gu, "gated_activation input", None, 2)
     T, two_i = gu.shape
     if two_i % 2:
         raise KernelError("gated_activation: the input needs an even number of columns")
     out = torch.empty((T, two_i // 2), dtype=gu.dtype, device=gu.device)
     if T:
-        _call("lc_gated_activation", _ptr(gu), _ptr(out), _dt(gu), T, two_i // 2, GATE_ACTIVATIONS[kind], _stream())
+        _call("lc_gated_activation", _ptr(gu), _ptr(out), _dt(gu), T, two_i // 2, 2 if form is not None else GATE_ACTIVATIONS[kind],
+              *((form.limit, form.slope, form.shift) if form is not None else (0.0, 0.0, 0.0)), _stream())
     return out
 
 
@@ -2041,4 +2083,123 @@ def scaled_sum(a, a_scale: float, b, b_scale: float) -> torch.Tensor:
     if out.numel():
         _call("lc_scaled_sum", _ptr(a), _dt(a), float(a_scale), _ptr(b), _dt(b), float(b_scale), _ptr(out),
               out.numel(), _stream())
+    return out
+
+
+def bias_add(x: torch.Tensor, bias: torch.Tensor) -> torch.Tensor:
+    """``x`` [T, n] plus ``bias`` float32 [n] in every row, rounded once to x's type."""
+    _need(x, "bias_add x", None, 2)
+    _need(bias, "bias_add bias", torch.float32, 1)
+    if bias.shape[0] != x.shape[1]:
+        raise KernelError(f"bias_add: {bias.shape[0]} entries for rows of {x.shape[1]}")
+    out = torch.empty_like(x)
+    if x.numel():
+        _call("lc_bias_add", _ptr(x), _dt(x), _ptr(bias), _ptr(out), x.shape[0], x.shape[1], _stream())
+    return out
+
+
+# ------------------------------------------------------------------------------ attention behind whole-row norms
+def attention_rows(proj: torch.Tensor, nq: int, nk: int, nv: int, d: int, dv: int, out_dtype: torch.dtype,
+                   k_cache: torch.Tensor, v_cache: torch.Tensor, rows: Optional[torch.Tensor],
+                   bias: Optional[torch.Tensor] = None, q_weight: Optional[torch.Tensor] = None,
+                   k_weight: Optional[torch.Tensor] = None, eps: float = 0.0, table: Optional[torch.Tensor] = None,
+                   rot: int = 0, half: bool = True, positions: Optional[torch.Tensor] = None,
+                   mix_from: Optional[torch.Tensor] = None, mix: float = 0.0, keep_values: bool = False):
+    """q for the attention kernels, and k and v into their cache rows, from the float32 projections ``proj`` [T,
+    cols]: columns q (nq heads of d) | k (nk of d) | v (nv of dv) | ....  ``bias`` float32 over these columns is
+    added first; ``q_weight`` [nq d] and ``k_weight`` [nk d]: all of a token's q (and all of its k) divided by its
+    root mean square (``eps`` inside the root) and weighed; ``table`` [positions, rot]: the first ``rot`` entries
+    of every q and k head are rotated, entry i with i + rot/2 (``half``) or 2i with 2i + 1.  ``mix_from`` float32
+    [T, nv dv]: v becomes (1 - mix) v + mix mix_from.  ``rows`` int32 [T]: the tokens' places in the cache
+    (page * page_size + offset; -1 or None: not written); ``k_cache`` [pages, page, nk d], ``v_cache`` [pages,
+    nv dv, page].  Returns (q [T, nq d] of ``out_dtype``, with ``keep_values`` v as it was before the mixing,
+    float32 [T, nv dv], else None)."""
+    _need(proj, "attention_rows proj", torch.float32, 2)
+    T, cols = proj.shape
+    C = (nq + nk) * d + nv * dv
+    if cols < C:
+        raise KernelError(f"attention_rows: {cols} columns, the heads need {C}")
+    _need(k_cache, "key cache", out_dtype, 3)
+    _need(v_cache, "value cache", out_dtype, 3)
+    page = k_cache.shape[1]
+    if k_cache.shape[2] != nk * d or v_cache.shape[1] != nv * dv or v_cache.shape[2] != page:
+        raise KernelError("attention_rows: the caches do not fit the heads")
+    for t, what, n in ((bias, "bias", C), (q_weight, "q weight", nq * d), (k_weight, "k weight", nk * d)):
+        if t is not None:
+            _need(t, f"attention_rows {what}", torch.float32, 1)
+            if t.shape[0] != n:
+                raise KernelError(f"attention_rows: the {what} has {t.shape[0]} entries, expected {n}")
+    if rows is not None:
+        _need(rows, "attention_rows rows", torch.int32, 1)
+        if rows.shape[0] != T:
+            raise KernelError("attention_rows: one place per token")
+    if table is not None:
+        _need(table, "rotary table", torch.float32, 2)
+        _need(positions, "positions", torch.int32, 1)
+        if table.shape[1] != rot or positions.shape[0] != T:
+            raise KernelError("attention_rows: the rotary table or the positions do not fit")
+    if mix_from is not None:
+        _need(mix_from, "attention_rows mixed-in values", torch.float32, 2)
+        if tuple(mix_from.shape) != (T, nv * dv):
+            raise KernelError(f"attention_rows: mixed-in values {tuple(mix_from.shape)}, expected {(T, nv * dv)}")
+    q = torch.empty((T, nq * d), dtype=out_dtype, device=proj.device)
+    values = torch.empty((T, nv * dv), dtype=torch.float32, device=proj.device) if keep_values else None
+    if T:
+        _call("lc_attention_rows", _ptr(proj), cols, T, nq, nk, nv, d, dv, _ptr(bias), _ptr(q_weight), _ptr(k_weight),
+              float(eps), _ptr(table), rot, 1 if half else 0, _ptr(positions), _ptr(mix_from), float(mix), _ptr(values),
+              _ptr(q), _ptr(k_cache), _ptr(v_cache), _dt(q), _ptr(rows), page, _stream())
+    return q, values
+
+
+# ------------------------------------------------------------------------------ matrix memory (mLSTM)
+def mlstm_prepare(proj: torch.Tensor, heads: int, key_dim: int, value_dim: int, i_column: int, f_column: int,
+                  i_bias: torch.Tensor, f_bias: torch.Tensor, cap: float, q_scale: float, reference: torch.Tensor,
+                  q_offsets: torch.Tensor, slot_ids: torch.Tensor, num_requests: int):
+    """The scan's inputs of the matrix memory from the float32 projections ``proj`` [T, cols]: columns q | k (heads
+    key_dim each) | v (heads value_dim) | ..., the gates' inputs at ``i_column`` and ``f_column`` (heads each).
+    i = cap tanh((x_i + i_bias) / cap), f = logsigmoid(cap tanh((x_f + f_bias) / cap)); from the request's
+    reference point m (``reference`` float32 [slots, heads], read at the slot before the request's first token of
+    the step, written after its last): m' = max(f + m, i).  Returns ``coef`` float32 [3, T, heads key_dim] (decay =
+    e^(f + m - m') in every channel, write = e^(i - m') k, read = q_scale q), ``v`` float32 [T, heads (value_dim +
+    1)] (a 1 behind every head's values: the channel of the normaliser) and ``bottoms`` float32 [T, heads], e^(-m')."""
+    _need(proj, "mlstm proj", torch.float32, 2)
+    T, cols = proj.shape
+    _need(i_bias, "mlstm i bias", torch.float32, 1)
+    _need(f_bias, "mlstm f bias", torch.float32, 1)
+    _need(reference, "mlstm reference points", torch.float32, 2)
+    _need(q_offsets, "q_offsets", torch.int32, 1)
+    _need(slot_ids, "slot_ids", torch.int32, 1)
+    if cols < heads * (2 * key_dim + value_dim) or i_bias.shape[0] != heads or f_bias.shape[0] != heads \
+            or reference.shape[1] != heads:
+        raise KernelError("mlstm_prepare: proj, the biases or the reference points do not fit the heads")
+    if q_offsets.shape[0] != num_requests + 1 or slot_ids.shape[0] != num_requests:
+        raise KernelError("mlstm_prepare: the request lists do not fit")
+    factors = torch.empty((3, T, heads), dtype=torch.float32, device=proj.device)
+    coef = torch.empty((3, T, heads * key_dim), dtype=torch.float32, device=proj.device)
+    v = torch.empty((T, heads * (value_dim + 1)), dtype=torch.float32, device=proj.device)
+    if T:
+        _call("lc_mlstm_prepare", _ptr(proj), cols, i_column, f_column, _ptr(i_bias), _ptr(f_bias), float(cap),
+              _ptr(reference), reference.shape[0], _ptr(q_offsets), _ptr(slot_ids), num_requests, T, heads, key_dim,
+              value_dim, float(q_scale), 1 if T == num_requests else 0, _ptr(factors), _ptr(coef), _ptr(v), _stream())
+    return coef, v, factors[2]
+
+
+def mlstm_readout(o: torch.Tensor, bottoms: torch.Tensor, floor: float, gates: torch.Tensor, gate_column: int,
+                  weight: torch.Tensor, eps: float, heads: int, value_dim: int, out_dtype: torch.dtype) -> torch.Tensor:
+    """``o`` float32 [T, heads (value_dim + 1)]: per head the memory's read-out and, last, the normaliser's.  Each
+    head's read-out over max(|normaliser|, ``bottoms``) + ``floor``, divided by its root mean square (``eps`` inside
+    the root), times ``weight`` [heads value_dim], times sigmoid of the float32 columns ``gate_column`` .. of
+    ``gates``.  -> [T, heads value_dim] of ``out_dtype``."""
+    _need(o, "mlstm_readout o", torch.float32, 2)
+    _need(bottoms, "mlstm_readout bottoms", torch.float32, 2)
+    _need(gates, "mlstm_readout gates", torch.float32, 2)
+    _need(weight, "mlstm_readout weight", torch.float32, 1)
+    T, n = o.shape[0], heads * value_dim
+    if o.shape[1] != heads * (value_dim + 1) or tuple(bottoms.shape) != (T, heads) or weight.shape[0] != n \
+            or gates.shape[0] != T or gate_column < 0 or gate_column + n > gates.shape[1]:
+        raise KernelError("mlstm_readout: o, the bottoms, the gates or the weight do not fit the heads")
+    out = torch.empty((T, n), dtype=out_dtype, device=o.device)
+    if T:
+        _call("lc_mlstm_readout", _ptr(o), _ptr(bottoms), float(floor), _ptr(gates), gates.shape[1], gate_column,
+              _ptr(weight), float(eps), T, heads, value_dim, _ptr(out), _dt(out), _stream())
     return out

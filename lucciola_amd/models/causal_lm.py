@@ -231,6 +231,7 @@ class CausalLM:
     # ------------------------------------------------------------------ forward
     def forward(self, batch: StepBatch, sites: List[SiteView]) -> torch.Tensor:
         """Run the batch's tokens through every site; float32 logits [wanted, vocab]."""
+        batch.passing.clear()
         if getattr(self.embed, "takes_positions", False):
             stream = ResidualStream(self.embed.forward(batch.token_ids, batch.positions))
         else:
@@ -245,6 +246,7 @@ class CausalLM:
             if index in self.before:
                 self.before[index].forward(stream)
             self.layers[entry.layer].block.forward(stream, sites[index])
+        batch.passing.clear()
         if batch.num_wanted == 0:
             return torch.empty((0, self.vocab_size), dtype=torch.float32, device=self.ctx.device)
         x = self.final_norm.add_norm_rows(stream, batch.want_rows)

@@ -1,7 +1,8 @@
 """The gated feed-forward (SwiGLU) as a part: ``down(silu(gate(x)) * up(x))``, no biases
 (reference: src/qwen.cc:762-794, src/kernels/swiglu.cu:8,31-35).  gate and up are one matrix
 product here: their weights are stacked at load.  The gate's activation is a parameter ("silu",
-or "gelu_tanh", which takes a kernel of its own behind the product)."""
+"gelu_tanh", which takes a kernel of its own behind the product, or "silu" in another form: both entries
+held below a ``limit``, a steeper sigmoid, the up entry shifted)."""
 from __future__ import annotations
 
 import math
@@ -32,11 +33,20 @@ class GatedMLP(Part):
     graph_safe = True   # launches only kernels whose arguments stay put between steps
     takes_scaled_rows = True   # x may be ops.ScaledRows; the output may be an ops.PendingProduct
 
-    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu"):
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu",
+                 limit: Optional[float] = None, slope: float = 1.0, shift: float = 0.0):
+        """``limit``, ``slope``, ``shift`` (with "silu"): with g' = min(gate, limit) and u' = up inside -limit ..
+        limit, the product is g' sigmoid(slope g') (u' + shift)."""
         super().__init__(hidden_size=hidden_size, intermediate_size=intermediate_size,
-                         activation=activation)
+                         activation=activation, limit=limit, slope=slope, shift=shift)
         if activation not in ops.GATE_ACTIVATIONS:
             raise ValueError(f"gated_mlp: activation '{activation}' has no kernel ({', '.join(ops.GATE_ACTIVATIONS)})")
+        form = ops.GateForm(float("inf") if limit is None else float(limit), float(slope), float(shift))
+        self.form = ops.SILU_GATE if form == ops.SILU_GATE else form
+        if self.form is not ops.SILU_GATE and activation != "silu":
+            raise ValueError("gated_mlp: limit, slope and shift go with 'silu'")
+        if not form.limit > 0:
+            raise ValueError(f"gated_mlp: the limit {limit} must be positive")
         self.H, self.I, self.activation = int(hidden_size), int(intermediate_size), activation
 
     def declare(self) -> Dict[str, ParamDecl]:
@@ -59,7 +69,9 @@ class GatedMLP(Part):
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         if self.fused:
-            z = ops.gemm_swiglu(x, self.gate_up)
+            z = ops.gemm_swiglu(x, self.gate_up, self.form)
+        elif self.form is not ops.SILU_GATE:
+            z = ops.gated_activation(ops.gemm(x, self.gate_up, self.dtype), self.activation, self.form)
         elif self.activation == "silu":
             z = ops.swiglu(ops.gemm(x, self.gate_up, self.dtype))
         else:

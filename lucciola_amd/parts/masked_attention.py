@@ -7,7 +7,14 @@
   divided by its root mean square over the value entries and multiplied by 1 - ``difference``;
 - ``conv_taps`` > 0: q, k and v pass a short causal convolution per channel right behind their projection
   (no bias, no activation); the last ``conv_taps`` - 1 projected rows of a request are state;
-- ``position``: a rotary encoding with interleaved pairs on the first entries of every map of every head;
+- ``position``: a rotary encoding on the first entries of every map of every head;
+- ``bias``: q, k and v and the output projection have biases;
+- ``row_norm``: all of a token's q, before it is split into heads, is divided by its root mean square and
+  multiplied by a weight of its size, and so is all of its k, before the rotation;
+- ``values``: the layer's values go to later layers or are mixed with an earlier layer's values of the same
+  token, (1 - lambda) v + lambda v_earlier with one learned number (tensor ``vmix``), before they are cached:
+  "keep": the values as projected stay for later layers of the pass; "mix": they are mixed with those that the last
+  "keep" layer before this one left (a "keep" layer has the tensor too and does not use it);
 - ``unit_qk``: every q and k head is divided by its root mean square (no weight);
 - ``distance_bias``: r1_h ln(1 + r2_h (i - j)) is taken off the score of query i and key j (two learned numbers a
   head);
@@ -16,8 +23,9 @@
 - ``chunk``: position i sees j <= i only inside its own chunk of that many positions, counted from the sequence's
   start; ``window``: only the last so many positions.
 
-The projections leave as float32; one kernel makes q, k and v of them (convolution, rotation, unit norm) and
-writes k and v into the cache (keys token-major, values transposed inside a page).  Scores, softmax, bias, sink
+The projections leave as float32; one kernel makes q, k and v of them (convolution, rotation of interleaved pairs,
+unit norm; or, with ``bias``, ``row_norm``, ``values`` or rotation of halves, the kernel that knows those:
+``ops.attention_rows``) and writes k and v into the cache (keys token-major, values transposed inside a page).  Scores, softmax, bias, sink
 and the maps' combination are float32 whatever the cache's type; with a bfloat16 cache of sizes that fit, the two
 products run on the matrix cores (``ops.masked_attention``), else in float32 multiply-adds.
 """
@@ -41,6 +49,9 @@ def _f32(t: torch.Tensor) -> torch.Tensor:
     return t.to(torch.float32).contiguous()
 
 
+PASSED_VALUES = "values"        # under which a "keep" layer leaves its values in the batch
+
+
 @MIXERS.register("masked_attention")
 class MaskedAttention(Part):
     graph_safe = True   # launches only kernels whose arguments stay put between steps
@@ -48,11 +59,13 @@ class MaskedAttention(Part):
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
                  scale: float, eps: float, maps: int = 1, difference: float = 0.0, conv_taps: int = 0,
                  position: Optional[PartSpec] = None, unit_qk: bool = False, distance_bias: bool = False,
-                 sink: bool = False, gate: bool = False, chunk: Optional[int] = None, window: Optional[int] = None):
+                 sink: bool = False, gate: bool = False, chunk: Optional[int] = None, window: Optional[int] = None,
+                 bias: bool = False, row_norm: bool = False, values: Optional[str] = None):
         super().__init__(hidden_size=hidden_size, num_heads=num_heads, num_kv_heads=num_kv_heads, head_dim=head_dim,
                          value_dim=value_dim, scale=scale, eps=eps, maps=maps, difference=difference,
                          conv_taps=conv_taps, position=position, unit_qk=unit_qk, distance_bias=distance_bias,
-                         sink=sink, gate=gate, chunk=chunk, window=window)
+                         sink=sink, gate=gate, chunk=chunk, window=window, bias=bias, row_norm=row_norm,
+                         values=values)
         if num_heads % num_kv_heads:
             raise ValueError(f"masked_attention: {num_heads} heads are not a multiple of {num_kv_heads} kv heads")
         if maps not in (1, 2):
@@ -70,9 +83,19 @@ class MaskedAttention(Part):
                                                                           bool(sink), bool(gate))
         self.chunk, self.window = int(chunk) if chunk else 0, int(window) if window else 0
         self.position = build_part(POSITION_ENCODINGS, position) if position else None
+        self.has_bias, self.row_norm, self.values = bool(bias), bool(row_norm), values
+        if values not in (None, "keep", "mix"):
+            raise ValueError(f"masked_attention: values '{values}' are neither 'keep' nor 'mix'")
+        pairing = getattr(self.position, "pairing", None)
+        if self.position is not None and pairing not in ("half", "interleaved"):
+            raise ValueError(f"masked_attention: no prologue kernel rotates with the pairing '{pairing}'")
+        self.half = pairing == "half"
+        # which of the two prologue kernels makes q, k and v
+        self.by_rows = self.has_bias or self.row_norm or self.values is not None or self.half
+        if self.by_rows and (self.taps or self.unit_qk):
+            raise ValueError("masked_attention: convolutions and unit_qk go without bias, row_norm, values and "
+                             "rotation of halves (no prologue kernel has both)")
         if self.position is not None:
-            if getattr(self.position, "pairing", None) != "interleaved":
-                raise ValueError("masked_attention: its kernel rotates entry 2i with entry 2i + 1 (pairing 'interleaved')")
             if self.position.rotary_dim > self.d:
                 raise ValueError(f"masked_attention: {self.position.rotary_dim} rotated entries in heads of {self.d}")
         self.nq_cols = self.nh * self.maps * self.d
@@ -97,6 +120,15 @@ class MaskedAttention(Part):
             out["sink"] = ParamDecl((self.nh,), role="vector")
         if self.has_gate:
             out["g"] = ParamDecl((self.nh * self.dv, self.H))
+        if self.has_bias:
+            for name, size in (("q_bias", self.nq_cols), ("k_bias", self.nk_cols), ("v_bias", self.nv_cols),
+                               ("o_bias", self.H)):
+                out[name] = ParamDecl((size,), role="vector")
+        if self.row_norm:
+            out["q_norm"] = ParamDecl((self.nq_cols,), role="vector", init="ones_plus_normal")
+            out["k_norm"] = ParamDecl((self.nk_cols,), role="vector", init="ones_plus_normal")
+        if self.values is not None:
+            out["vmix"] = ParamDecl((), role="vector")
         return out
 
     def bind(self, tensors, ctx: BuildContext) -> None:
@@ -115,6 +147,14 @@ class MaskedAttention(Part):
         self.r1 = _f32(tensors["r1"]) if self.distance_bias else None
         self.r2 = _f32(tensors["r2"]) if self.distance_bias else None
         self.sink = _f32(tensors["sink"]) if self.has_sink else None
+        self.bias = self.o_bias = self.q_norm = self.k_norm = None
+        if self.has_bias:
+            self.bias = torch.cat([_f32(tensors[k]) for k in ("q_bias", "k_bias", "v_bias")]).contiguous()
+            self.o_bias = _f32(tensors["o_bias"])
+        if self.row_norm:
+            self.q_norm, self.k_norm = _f32(tensors["q_norm"]), _f32(tensors["k_norm"])
+        # one number for the layer; read once, at load
+        self.mix = float(tensors["vmix"].to(torch.float32).item()) if self.values == "mix" else 0.0
         if self.position is not None:
             self.position.bind({}, ctx)
 
@@ -144,7 +184,7 @@ class MaskedAttention(Part):
         table, rot = None, 0
         if self.position is not None:
             table, rot = self.position.rotary_table(batch.max_position), self.position.rotary_dim
-        q = ops.attention_prepare(
+        q = self._by_rows(proj, site, k_cache, v_cache, table, rot) if self.by_rows else ops.attention_prepare(
             proj, self.nh * self.maps, self.nkv * self.maps, self.nkv, self.d, self.dv, self.dtype,
             k_cache, v_cache, pages.slots if site.writes_cache else None,
             taps=self.conv, tail=tail, tok_req=batch.tok_req, q_offsets=batch.q_offsets, slot_ids=batch.slot_ids,
@@ -159,4 +199,20 @@ class MaskedAttention(Part):
             out_scale=1.0 - self.difference if self.maps == 2 else 1.0,
             gate=proj if self.has_gate else None, gate_column=self.channels, plan=batch.plans.get(ops.LATENT_PLAN),
             max_ctx=batch.max_ctx)
-        return ops.gemm(o, self.o, self.dtype, defer=True)
+        y = ops.gemm(o, self.o, self.dtype, defer=True)
+        return ops.BiasedBranch(y, self.o_bias) if self.has_bias else y
+
+    def _by_rows(self, proj: torch.Tensor, site, k_cache, v_cache, table, rot: int) -> torch.Tensor:
+        batch, earlier = site.batch, None
+        if self.values == "mix":
+            earlier = batch.passing.get(PASSED_VALUES)
+            if earlier is None:
+                raise ValueError("masked_attention: no earlier layer has left values to mix in")
+        q, own = ops.attention_rows(
+            proj, self.nh * self.maps, self.nkv * self.maps, self.nkv, self.d, self.dv, self.dtype, k_cache, v_cache,
+            site.part(0).pages.slots if site.writes_cache else None, bias=self.bias, q_weight=self.q_norm,
+            k_weight=self.k_norm, eps=self.eps, table=table, rot=rot, half=self.half, positions=batch.positions,
+            mix_from=earlier, mix=self.mix, keep_values=self.values == "keep")
+        if own is not None:
+            batch.passing[PASSED_VALUES] = own
+        return q

@@ -18,21 +18,26 @@ class RMSNorm(Part):
     graph_safe = True   # launches only kernels whose arguments stay put between steps
     offers_scaled_rows = True   # add_norm(stream, scaled=True) may return ops.ScaledRows
 
-    def __init__(self, size: int, eps: float, scalar: bool = False):
-        super().__init__(size=size, eps=eps, scalar=scalar)
+    def __init__(self, size: int, eps: float, scalar: bool = False, one_plus: bool = False):
+        super().__init__(size=size, eps=eps, scalar=scalar, one_plus=one_plus)
         self.size, self.eps = int(size), float(eps)
         # scalar: the learned weight is one number for all coordinates (``gain``); the kernels still
         # get a vector, that number in every entry
         self.scalar = bool(scalar)
+        # one_plus: the weight is stored around zero, the row is multiplied by 1 + weight (added once, at load)
+        self.one_plus = bool(one_plus)
         self.gain: Optional[float] = None
         self.weight: Optional[torch.Tensor] = None
         self.dtype = None
 
     def declare(self) -> Dict[str, ParamDecl]:
-        return {"weight": ParamDecl(() if self.scalar else (self.size,), role="vector", init="ones_plus_normal")}
+        return {"weight": ParamDecl(() if self.scalar else (self.size,), role="vector",
+                                    init="normal" if self.one_plus else "ones_plus_normal")}
 
     def bind(self, tensors, ctx: BuildContext) -> None:
         self.weight = tensors["weight"]
+        if self.one_plus:
+            self.weight = (self.weight.to(torch.float32) + 1.0).contiguous()
         if self.scalar:
             self.gain = float(self.weight.to(torch.float32).item())     # a kernel argument; read once, at load
             self.weight = self.weight.to(torch.float32).reshape(1).expand(self.size).contiguous()

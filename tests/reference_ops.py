@@ -17,6 +17,8 @@ def embedding(ids, table, scale=1.0):
 
 
 def rmsnorm(h, delta, weight, eps, out_dtype, rows=None, scaled=False):   # never hands out scaled rows
+    if hasattr(delta, "branch"):            # a branch and its bias
+        delta = delta.branch.to(F64) + delta.bias.to(F64)
     if rows is None:
         if delta is not None:
             h += delta.to(torch.float32)
@@ -387,9 +389,12 @@ def embedding_sinusoid(ids, table, positions, frequencies, scale=1.0):
     return out
 
 
-def gated_activation(gu, kind):
+def gated_activation(gu, kind, form=None):
     I = gu.shape[1] // 2
     g, u = gu[:, :I].to(F64), gu[:, I:].to(F64)
+    if form is not None:
+        g, u = torch.clamp(g, max=form.limit), torch.clamp(u, min=-form.limit, max=form.limit)
+        return (g / (1 + torch.exp(-form.slope * g)) * (u + form.shift)).to(gu.dtype)
     a = g / (1 + torch.exp(-g)) if kind == "silu" else _act(g, kind)
     return (a * u).to(gu.dtype)
 
@@ -659,6 +664,73 @@ def scaled_sum(a, a_scale, b, b_scale):
     return (a_scale * a.to(F64) + b_scale * b.to(F64)).to(torch.float32)
 
 
+def bias_add(x, bias):
+    return (x.to(F64) + bias.to(F64)).to(x.dtype)
+
+
+def attention_rows(proj, nq, nk, nv, d, dv, out_dtype, k_cache, v_cache, rows, bias=None, q_weight=None, k_weight=None,
+                   eps=0.0, table=None, rot=0, half=True, positions=None, mix_from=None, mix=0.0, keep_values=False):
+    T = proj.shape[0]
+    C = (nq + nk) * d + nv * dv
+    y = proj[:, :C].to(F64)
+    if bias is not None:
+        y = y + bias.to(F64)
+    q, k, v = y[:, :nq * d], y[:, nq * d:(nq + nk) * d], y[:, (nq + nk) * d:]
+    if q_weight is not None:
+        q = q / torch.sqrt((q * q).mean(-1, keepdim=True) + eps) * q_weight.to(F64)
+        k = k / torch.sqrt((k * k).mean(-1, keepdim=True) + eps) * k_weight.to(F64)
+    qk = torch.cat([q, k], dim=1).reshape(T, nq + nk, d)
+    if table is not None:
+        cs = table[positions.long()].to(F64)
+        cos, sin = cs[:, None, :rot // 2], cs[:, None, rot // 2:]
+        one, other = (slice(0, rot // 2), slice(rot // 2, rot)) if half else (slice(0, rot, 2), slice(1, rot, 2))
+        a, b = qk[..., one].clone(), qk[..., other].clone()
+        qk[..., one] = a * cos - b * sin
+        qk[..., other] = b * cos + a * sin
+    values = v.to(torch.float32) if keep_values else None
+    if mix_from is not None:
+        v = (1 - mix) * v + mix * mix_from.to(F64)
+    if rows is not None:
+        page = k_cache.shape[1]
+        keep = rows >= 0
+        at = rows[keep].long()
+        k_cache[at // page, at % page] = qk[keep, nq:].reshape(-1, nk * d).to(k_cache.dtype)
+        v_cache[at // page, :, at % page] = v[keep].to(v_cache.dtype)
+    return qk[:, :nq].reshape(T, nq * d).to(out_dtype), values
+
+
+def mlstm_prepare(proj, heads, key_dim, value_dim, i_column, f_column, i_bias, f_bias, cap, q_scale, reference, q_offsets,
+                  slot_ids, num_requests):
+    T, nk = proj.shape[0], heads * key_dim
+    p = proj.to(F64)
+    log_in = cap * torch.tanh((p[:, i_column:i_column + heads] + i_bias.to(F64)) / cap)
+    log_keep = torch.nn.functional.logsigmoid(cap * torch.tanh((p[:, f_column:f_column + heads] + f_bias.to(F64)) / cap))
+    keep, write, bottom = (torch.zeros(T, heads, dtype=F64) for _ in range(3))
+    starts = q_offsets.tolist()
+    for r in range(num_requests):
+        m = reference[int(slot_ids[r])].to(F64)
+        for t in range(starts[r], starts[r + 1]):
+            after = torch.maximum(log_keep[t] + m, log_in[t])
+            keep[t], write[t], bottom[t] = torch.exp(log_keep[t] + m - after), torch.exp(log_in[t] - after), torch.exp(-after)
+            m = after
+        reference[int(slot_ids[r])] = m.to(reference.dtype)
+    q, k = p[:, :nk].view(T, heads, key_dim), p[:, nk:2 * nk].view(T, heads, key_dim)
+    coef = torch.stack([keep[:, :, None].expand(T, heads, key_dim), write[:, :, None] * k, q_scale * q])
+    v = torch.ones(T, heads, value_dim + 1, dtype=F64)
+    v[:, :, :value_dim] = p[:, 2 * nk:2 * nk + heads * value_dim].view(T, heads, value_dim)
+    return (coef.reshape(3, T, nk).to(torch.float32).contiguous(),
+            v.view(T, -1).to(torch.float32).contiguous(), bottom.to(torch.float32))
+
+
+def mlstm_readout(o, bottoms, floor, gates, gate_column, weight, eps, heads, value_dim, out_dtype):
+    T, n = o.shape[0], heads * value_dim
+    x = o.to(F64).view(T, heads, value_dim + 1)
+    x = x[:, :, :value_dim] / (torch.maximum(x[:, :, value_dim:].abs(), bottoms.to(F64)[:, :, None]) + floor)
+    x = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+    g = torch.sigmoid(gates[:, gate_column:gate_column + n].to(F64))
+    return (x.reshape(T, n) * weight.to(F64) * g).to(out_dtype)
+
+
 def moe_large_tiles(x_dtype, up, down):
     return False
 
@@ -670,7 +742,7 @@ ALL = ("layer_norm", "layer_norm_act", "embedding_sinusoid", "gated_activation",
        "latent_prepare", "latent_attention", "moe_route", "moe_experts", "moe_combine",
        "scale_", "token_shift", "rms_shift", "moe_route_sigmoid", "lightning_prepare", "lightning_readout",
        "gated_activation_weighted", "attention_prepare", "masked_attention", "state_space_prepare",
-       "state_space_readout", "scaled_sum")
+       "state_space_readout", "scaled_sum", "bias_add", "attention_rows", "mlstm_prepare", "mlstm_readout")
 
 
 def install(monkeypatch):
