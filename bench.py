@@ -434,6 +434,22 @@ def rununex_design_config(name, routed=True):
             "initializer_range": 0.02, "layers": layers}
 
 
+def vasanex_design_config(name, routed=False):
+    """The Vasanex decoder at the same width, heads, head size, feed-forward width, vocabulary and depth: attention
+    (heads of 128 over heads / 4 key/value heads, biases, whole-row norms, half of each head's entries rotated, window
+    4,096, a sink, mixed values) and the mLSTM's matrix memory (heads of 128 x 128) in turn, a dense gated
+    feed-forward in every layer."""
+    width, heads, ff = DESIGN_SIZES[name]
+    attention = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                 "mask": {"size": 4096}, "rot": {"base": 500000.0, "dims": 64}, "v_mix": True}
+    memory = {"heads": heads, "dim": 128, "vdim": 128, "gate_cap": 15.0}
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    layers = [{"type": "attention", "mixer": attention, "mlp": dense}, {"type": "mlstm", "mixer": memory, "mlp": dense},
+              {"type": "attention", "mixer": attention, "mlp": dense}, {"type": "mlstm", "mixer": memory, "mlp": dense}]
+    return {"architecture": "Vasanex", "vocab": DESIGN_VOCAB, "width": width, "norm": {"eps": 1e-6},
+            "embedding": {"scale": 2.0}, "initializer_range": 0.02, "layers": layers}
+
+
 def design_run(cfg, dtype, dev, block_size, prompt, batches, context, steps):
     """Prompt and decode throughput of one configuration through the runner's own step."""
     import torch
@@ -516,10 +532,11 @@ def designs_workload(args, dev):
                 results[key] = design_run(pubodra, dtype, dev, args.block_size, args.prefill_tokens, batches,
                                           args.design_context, args.steps)
                 say(f"{key}: {results[key]}")
-        for model in ("larupel", "larupel_dense", "kikunex", "kikunex_dense", "rununex", "rununex_dense"):
+        for model in ("larupel", "larupel_dense", "kikunex", "kikunex_dense", "rununex", "rununex_dense", "vasanex"):
             if model in wanted:
                 key = f"{name}/{model}"
-                make = {"l": larupel_design_config, "k": kikunex_design_config, "r": rununex_design_config}[model[0]]
+                make = {"l": larupel_design_config, "k": kikunex_design_config, "r": rununex_design_config,
+                        "v": vasanex_design_config}[model[0]]
                 results[key] = design_run(make(name, routed="dense" not in model), dtype, dev,
                                           args.block_size, args.prefill_tokens, batches, args.design_context, args.steps)
                 say(f"{key}: {results[key]}")
@@ -571,7 +588,7 @@ def main() -> int:
     ap.add_argument("--design-batches", default="8,64", help="designs: decode batch sizes")
     ap.add_argument("--design-models", default="qwen3,pubodra_dense,pubodra_routed,larupel",
                     help="designs: which of qwen3, pubodra_dense, pubodra_routed, larupel, larupel_dense, kikunex, kikunex_dense, "
-                         "rununex, rununex_dense")
+                         "rununex, rununex_dense, vasanex")
     ap.add_argument("--design-context", type=int, default=2048, help="designs: tokens a decoding request holds")
     ap.add_argument("--workload", default="decode", choices=["decode", "mixed", "designs"],
                     help="decode: the default line; mixed: only the 0.6B-shaped mixed workload, as a line of its own")

@@ -16,19 +16,25 @@
 
 namespace lc {
 
-// What the token's gates make of the reference point before it.
+// What the token's gates make of the reference point before it.  The kernel of lone tokens and the one that walks a
+// portion both go through these; a multiplication is not taken into a following addition, so that they give the same bits.
 struct MemoryGates {
     float keep_log, write_log;
 };
 __device__ __forceinline__ MemoryGates memory_gates(float x_i, float b_i, float x_f, float b_f, float cap) {
+#pragma clang fp contract(off)
     const float z = cap * tanhf((x_f + b_f) / cap);
     return {fminf(z, 0.f) - log1pf(expf(-fabsf(z))), cap * tanhf((x_i + b_i) / cap)};
 }
 __device__ __forceinline__ float next_reference(const MemoryGates& g, float m) { return fmaxf(g.keep_log + m, g.write_log); }
 __device__ __forceinline__ float keep_factor(const MemoryGates& g, float before, float after) {
+#pragma clang fp contract(off)
     return expf(g.keep_log + before - after);
 }
-__device__ __forceinline__ float write_factor(const MemoryGates& g, float after) { return expf(g.write_log - after); }
+__device__ __forceinline__ float write_factor(const MemoryGates& g, float after) {
+#pragma clang fp contract(off)
+    return expf(g.write_log - after);
+}
 
 __device__ __forceinline__ float from_lane(float v, int lane) {
     return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane));
