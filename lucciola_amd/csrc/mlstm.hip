@@ -6,7 +6,7 @@
 // The normaliser is one more value channel, whose value is 1 in every token: with it beside the others the
 // recurrence is S <- diag(decay) S + write v^T, o = S^T read without a removal term, with decay = e^(f + m - m') in
 // every key channel, write = e^(i - m') k, read = q_scale q.  This file makes those inputs from a step's float32
-// projections: the reference points, which tie a token to the one before it, by one wave per request and head that
+// projections: the reference points, which tie a token to the one before it, by one workgroup per request and head that
 // walks the request's tokens; the vectors by a thread an entry.  A step of lone tokens does both in one kernel.
 // Behind the scan the read-out divides by the normaliser, takes each head by its root mean square, multiplies by a
 // weight and sigmoid(gate) and rounds to the activation type; everything before that rounding is float32.
@@ -36,53 +36,81 @@ __device__ __forceinline__ float write_factor(const MemoryGates& g, float after)
     return expf(g.write_log - after);
 }
 
-__device__ __forceinline__ float from_lane(float v, int lane) {
-    return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane));
-}
+constexpr int GATE_TOKENS = 192;       // tokens of a chunk: one for each thread behind the first wave
+constexpr int CHAIN_GROUP = 16;         // tokens that the walker reads ahead
 
-// grid (heads, requests), one wave.  proj [T, cols] with x_i at columns i_col + head and x_f at f_col + head;
-// factors [3, T, heads]: keep, write and e^(-m') of every token; reference [slots, heads].
-// 64 tokens at a time: their gates side by side, then the chain of maxima, one add and one max a token, in order, so
-// that a token's numbers have the same bits however its request is cut into steps.
-__global__ __launch_bounds__(kWave) void mlstm_gates_kernel(
+// grid (heads, requests).  proj [T, cols] with x_i at columns i_col + head and x_f at f_col + head; factors
+// [3, T, heads]: keep, write and e^(-m') of every token; reference [slots, heads].
+// A pipeline over chunks of tokens: while the other waves make the gates of chunk c (a token a thread) and write out
+// chunk c - 2, one lane of the first wave walks the chain of maxima through chunk c - 1, one add and one max a token,
+// in order, so that a token's numbers have the same bits however its request is cut into steps.
+__global__ __launch_bounds__(kWave + GATE_TOKENS) void mlstm_gates_kernel(
     const float* __restrict__ proj, int cols, int i_col, int f_col, const float* __restrict__ i_bias,
     const float* __restrict__ f_bias, float cap, float* __restrict__ reference, const int* __restrict__ q_offsets,
     const int* __restrict__ slot_ids, int T, int heads, float* __restrict__ factors) {
-    const int head = blockIdx.x, req = blockIdx.y, lane = threadIdx.x;
+    static_assert(GATE_TOKENS % CHAIN_GROUP == 0 && CHAIN_GROUP % 4 == 0, "whole groups of whole float4s");
+    __shared__ float4 keep_log[2][GATE_TOKENS / 4], write_log[2][GATE_TOKENS / 4], found[2][GATE_TOKENS / 4];
+    const int head = blockIdx.x, req = blockIdx.y, j = (int)threadIdx.x - kWave;
     const int first = q_offsets[req], last = q_offsets[req + 1];
-    float* home = reference + (size_t)slot_ids[req] * heads + head;
+    if (first >= last) return;
+    const int chunks = (last - first + GATE_TOKENS - 1) / GATE_TOKENS;
     const size_t plane = (size_t)T * heads;
+    float* home = reference + (size_t)slot_ids[req] * heads + head;
     const float b_i = i_bias[head], b_f = f_bias[head];
     float m = *home;
-    auto fetch = [&](int t0, float& x_i, float& x_f) {
-        const int t = min(t0 + lane, last - 1);
-        x_i = proj[(size_t)t * cols + i_col + head];
-        x_f = proj[(size_t)t * cols + f_col + head];
-    };
-    float x_i = 0.f, x_f = 0.f;
-    if (first < last) fetch(first, x_i, x_f);
-    for (int t0 = first; t0 < last; t0 += kWave) {
-        const int count = min(kWave, last - t0);
-        MemoryGates g = memory_gates(x_i, b_i, x_f, b_f, cap);
-        if (t0 + kWave < last) fetch(t0 + kWave, x_i, x_f);     // on their way during the chain
-        if (lane >= count) g = {0.f, -INFINITY};                // behind the request's end: nothing moves
-        const float entry = m;
-        float after = m;
+    for (int c = 0; c < chunks + 2; ++c) {
+        const int mine = c & 1, walked = mine ^ 1;      // the chunks c and c - 2 share their places
+        if (j >= 0) {
+            if (c >= 2) {
+                const int t = first + (c - 2) * GATE_TOKENS + j;
+                if (t < last) {
+                    const MemoryGates g{((const float*)keep_log[mine])[j], ((const float*)write_log[mine])[j]};
+                    const float before = ((const float*)found[mine])[j], after = next_reference(g, before);
+                    const size_t at = (size_t)t * heads + head;
+                    factors[at] = keep_factor(g, before, after);
+                    factors[plane + at] = write_factor(g, after);
+                    factors[2 * plane + at] = expf(-after);
+                }
+            }
+            if (c < chunks) {
+                const int t = first + c * GATE_TOKENS + j;
+                MemoryGates g = {0.f, -INFINITY};       // behind the request's end: nothing moves
+                if (t < last) {
+                    const float* row = proj + (size_t)t * cols;
+                    g = memory_gates(row[i_col + head], b_i, row[f_col + head], b_f, cap);
+                }
+                ((float*)keep_log[mine])[j] = g.keep_log;
+                ((float*)write_log[mine])[j] = g.write_log;
+            }
+        } else if (threadIdx.x == 0 && c >= 1 && c <= chunks) {
+            constexpr int QUADS = CHAIN_GROUP / 4;
+            const float4 *keep = keep_log[walked], *write = write_log[walked];
+            const int count = min(GATE_TOKENS, last - first - (c - 1) * GATE_TOKENS);
+            const int groups = (count + CHAIN_GROUP - 1) / CHAIN_GROUP;
+            float4 k_now[QUADS], w_now[QUADS], k_next[QUADS], w_next[QUADS];
 #pragma unroll
-        for (int k = 0; k < kWave; ++k) {
-            m = fmaxf(from_lane(g.keep_log, k) + m, from_lane(g.write_log, k));
-            after = lane == k ? m : after;
+            for (int i = 0; i < QUADS; ++i) k_now[i] = keep[i], w_now[i] = write[i];
+            for (int n = 0; n < groups; ++n) {
+                const int ahead = min(n + 1, groups - 1) * QUADS;
+#pragma unroll
+                for (int i = 0; i < QUADS; ++i) k_next[i] = keep[ahead + i], w_next[i] = write[ahead + i];
+#pragma unroll
+                for (int i = 0; i < QUADS; ++i) {
+                    float4 at;
+                    at.x = m;
+                    at.y = next_reference({k_now[i].x, w_now[i].x}, at.x);
+                    at.z = next_reference({k_now[i].y, w_now[i].y}, at.y);
+                    at.w = next_reference({k_now[i].z, w_now[i].z}, at.z);
+                    m = next_reference({k_now[i].w, w_now[i].w}, at.w);
+                    found[walked][n * QUADS + i] = at;
+                }
+#pragma unroll
+                for (int i = 0; i < QUADS; ++i) k_now[i] = k_next[i], w_now[i] = w_next[i];
+            }
+            if (c == chunks) *home = m;
         }
-        float before = __shfl_up(after, 1, kWave);
-        if (lane == 0) before = entry;
-        if (lane < count) {
-            const size_t at = (size_t)(t0 + lane) * heads + head;
-            factors[at] = keep_factor(g, before, after);
-            factors[plane + at] = write_factor(g, after);
-            factors[2 * plane + at] = expf(-after);
-        }
+        __syncthreads();
     }
-    if (lane == 0 && first < last) *home = m;
 }
 
 // A thread per entry.  proj [T, cols]: q | k (heads x dk each) | v (heads x dv) | ...; coef [3, T, heads dk]: decay,
@@ -193,7 +221,7 @@ LC_API int lc_mlstm_prepare(const float* proj, int cols, int i_col, int f_col, c
         LC_LAUNCH_CHECK("mlstm_lone");
         return 0;
     }
-    mlstm_gates_kernel<<<dim3(heads, R), kWave, 0, stream>>>(proj, cols, i_col, f_col, i_bias, f_bias, cap, reference,
+    mlstm_gates_kernel<<<dim3(heads, R), kWave + GATE_TOKENS, 0, stream>>>(proj, cols, i_col, f_col, i_bias, f_bias, cap, reference,
                                                              q_offsets, slot_ids, T, heads, factors);
     LC_LAUNCH_CHECK("mlstm_gates");
     const size_t total = (size_t)T * heads * (dk + dv + 1);

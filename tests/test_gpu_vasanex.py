@@ -100,17 +100,20 @@ ROWS_CASES = [
     (4, 1, 1, 64, 16, 16, 9, 10, False, True, False, None),
     (6, 2, 2, 12, 20, 8, 33, 12, False, False, True, "mix"),
     (2, 1, 1, 256, 256, 16, 2, 2, True, False, False, "keep"),
+    (5, 1, 1, 24, 12, 4, 6, 12, False, True, True, "mix"),
+    (8, 4, 4, 80, 36, 16, 40, 40, True, True, True, "keep"),
 ]
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("case_", ROWS_CASES)
-def test_attention_rows(case_, dtype):
+@pytest.mark.parametrize("extra", [5, 8])       # columns behind the heads: with 5, rows begin at odd places
+def test_attention_rows(case_, dtype, extra):
     """q, the cache rows (and every row that is not a token's: untouched) and the kept values."""
     nq, nk, nv, d, dv, page, T, rot, half, bias, norm, values = case_
     g = torch.Generator().manual_seed(nq * 100 + d)
     C = (nq + nk) * d + nv * dv
-    proj = torch.randn(T, C + 5, generator=g) * 2
+    proj = torch.randn(T, C + extra, generator=g) * 2
     pages = T // page + 4
     places = torch.randperm(pages * page, generator=g)[:T].to(torch.int32)
     places[T // 2] = -1 if T > 2 else places[T // 2]
@@ -208,9 +211,9 @@ MEMORY_CASES = [
     # heads, dk, dv, cap, lengths of two steps
     (4, 32, 48, 12.0, [70, 1, 129, 2]),
     (3, 7, 5, 2.5, [3, 200, 1, 64]),
-    (1, 128, 128, 15.0, [65, 300, 1, 5]),
+    (1, 128, 128, 15.0, [65, 600, 1, 193]),
     (2, 16, 16, 6.0, [1, 1, 1, 1]),
-    (5, 64, 31, 0.7, [63, 64, 2, 1]),
+    (5, 64, 31, 0.7, [191, 192, 2, 385]),
     (2, 256, 8, 9.0, [1, 1, 40, 1]),
 ]
 
@@ -252,8 +255,8 @@ def test_matrix_memory_kernels(case_):
 
 
 def test_reference_points_have_the_same_bits_for_every_cut():
-    """150 tokens whole, in portions and one by one (the kernel of lone tokens): gates, reads and reference points."""
-    heads, dk, dv, T = 3, 8, 8, 150
+    """450 tokens whole, in portions and one by one (the kernel of lone tokens): gates, reads and reference points."""
+    heads, dk, dv, T = 3, 8, 8, 450
     g = torch.Generator().manual_seed(5)
     cols = heads * (2 * dk + dv) + 2 * heads
     proj = (torch.randn(T, cols, generator=g) * 3).to(DEV)
@@ -269,7 +272,7 @@ def test_reference_points_have_the_same_bits_for_every_cut():
         return [torch.cat([p[0] for p in parts], dim=1), torch.cat([p[1] for p in parts]),
                 torch.cat([p[2] for p in parts]), reference]
     whole = run(T)
-    for cut in (1, 2, 63, 64, 65, 100):
+    for cut in (1, 2, 15, 63, 100, 191, 192, 193, 385):
         for a, b in zip(whole, run(cut)):
             assert torch.equal(a, b), f"portions of {cut}: the bits differ"
 
