@@ -196,7 +196,7 @@ LC_API int lc_attention_rows(const float* proj, int cols, int T, int nq, int nk,
     LC_CHECK((q_weight == nullptr) == (k_weight == nullptr), "attention rows: q and k are normed together");
     LC_CHECK(!table || (rot > 0 && rot % 2 == 0 && rot <= d && positions), "attention rows: bad rotation");
     LC_CHECK(!rows || (k_cache && v_cache && page_size > 0), "attention rows: rows without a cache");
-    // few tokens: several workgroups a token, so that the card is not left to a handful of them
+    // few tokens: several workgroups a token, so that the GPU is not left to a handful of them
     const bool quads = d % 4 == 0 && dv % 4 == 0 && cols % 4 == 0 && (!table || rot % (half ? 8 : 4) == 0) &&
                        in_sixteens(proj) && in_sixteens(bias) && in_sixteens(q_weight) && in_sixteens(k_weight) &&
                        in_sixteens(table) && in_sixteens(mix_from) && in_sixteens(values_out) && in_sixteens(q_out) &&

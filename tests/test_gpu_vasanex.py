@@ -209,7 +209,7 @@ def test_one_key_carries_the_weight_at_a_windows_edges(dtype, window):
 
 MEMORY_CASES = [
     # heads, dk, dv, cap, lengths of two steps
-    (4, 32, 48, 12.0, [70, 1, 129, 2]),
+    (4, 32, 40, 11.0, [70, 1, 129, 2]),
     (3, 7, 5, 2.5, [3, 200, 1, 64]),
     (1, 128, 128, 15.0, [65, 600, 1, 193]),
     (2, 16, 16, 6.0, [1, 1, 1, 1]),
