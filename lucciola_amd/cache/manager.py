@@ -6,7 +6,8 @@ need counts its own bytes and makes its own memory, the manager keeps the books.
 Sites with equal paged needs form a *group*: one pool of page ids and one block table per
 request serve the whole group, and each site of the group has key and value tensors of its
 own that are indexed by those page ids.  Groups differ in what they keep: all keys, or a
-window of them, in which case the pages the window has passed are given back after each step.
+window of them (and the first few beside it), in which case the pages the window has passed are given back after
+each step.
 
 The reference has one group (every layer alike, src/qwen.cc:507-516), takes a page when
 ``ceil(len / block_size)`` exceeds the table (src/scheduler.cc:55-58,89-97) and gives all of
@@ -206,7 +207,8 @@ class CacheManager:
             # the next query is at position >= length and reads keys > position - w
             first_needed = st.length - w + 1
             table = g.tables[request]
-            for idx in range(min(len(table), max(0, first_needed // self.block_size))):
+            kept = _ceil_div(g.spec.keep_first, self.block_size)        # pages that hold first positions stay
+            for idx in range(kept, min(len(table), max(0, first_needed // self.block_size))):
                 if table[idx] >= 0:
                     g.pool.free(table[idx])
                     table[idx] = -1

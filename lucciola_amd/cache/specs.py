@@ -47,6 +47,7 @@ class CacheNeed:
 
     paged = False
     window: Optional[int] = None    # paged: only the last ``window`` positions are read again
+    keep_first: int = 0             # paged, beside a window: and the first so many positions
 
     def kernel_page(self, page_size: int) -> int:
         """Tokens of a page as this need's kernels index it, for the manager's page size: a
@@ -124,7 +125,8 @@ class PagedLatent(CacheNeed):
 class PagedRows(CacheNeed):
     """A row of keys and a row of values per token, in pages, the two of widths of their own (key heads and
     value heads of different numbers or sizes, several key maps that share a value).  ``window`` as for
-    :class:`PagedKV`.
+    :class:`PagedKV`; the first ``keep_first`` positions are read again whatever the window has passed, so
+    their pages stay.
 
     Memory per site: keys token-major ``[pages, page, key_width]``, values transposed inside a page ``[pages,
     value_width, page]`` (a matrix-core operand wants a value entry's neighbouring positions side by side); any
@@ -133,6 +135,7 @@ class PagedRows(CacheNeed):
     key_width: int
     value_width: int
     window: Optional[int] = None
+    keep_first: int = 0
 
     paged = True
 

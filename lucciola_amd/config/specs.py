@@ -62,6 +62,16 @@ def prenorm_layer(mixer: PartSpec, feed_forward: PartSpec, mixer_norm: PartSpec,
                       "feed_forward_norm": feed_forward_norm}, names)
 
 
+def parallel_layer(mixer: PartSpec, feed_forward: Optional[PartSpec], mixer_norm: PartSpec,
+                   feed_forward_norm: Optional[PartSpec], names: Dict[str, str]) -> LayerSpec:
+    """A layer whose mixer and feed-forward read the same stream, each behind its own norm (``parallel_residual``, or
+    ``parallel_mixer`` without a feed-forward)."""
+    if feed_forward is None:
+        return LayerSpec("parallel_mixer", {"mixer": mixer, "mixer_norm": mixer_norm}, names)
+    return LayerSpec("parallel_residual", {"mixer": mixer, "feed_forward": feed_forward, "mixer_norm": mixer_norm,
+                                           "feed_forward_norm": feed_forward_norm}, names)
+
+
 @dataclass(frozen=True)
 class RunEntry:
     """One entry of the run order: run ``layer`` here.

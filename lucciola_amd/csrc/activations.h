@@ -9,13 +9,14 @@ namespace lc {
 // ACT_SIGMOID_GATE: times sigmoid of the gate's entry at the output's place; ACT_SIGMOID_GROUP_GATE: times
 // sigmoid of ONE gate entry per row and group (a number per token and head)
 enum : int { ACT_NONE = 0, ACT_GELU_TANH = 1, ACT_RELU_SQUARED = 2, ACT_SIGMOID_GATE = 3, ACT_SIGMOID_GROUP_GATE = 4,
-             ACT_XIELU = 5 };
+             ACT_XIELU = 5, ACT_GELU_ERF = 6 };
 
 __device__ __forceinline__ float activate(float z, int kind) {
     if (kind == ACT_GELU_TANH) {
         const float inner = 0.7978845608028654f * fmaf(0.044715f * z, z * z, z);   // sqrt(2/pi) (z + 0.044715 z^3)
         return 0.5f * z * (1.f + tanhf(inner));
     }
+    if (kind == ACT_GELU_ERF) return 0.5f * z * (1.f + erff(z * 0.7071067811865476f));
     if (kind == ACT_RELU_SQUARED) {
         const float r = fmaxf(z, 0.f);
         return r * r;

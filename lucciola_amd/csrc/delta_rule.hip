@@ -17,6 +17,7 @@
 //   gated         q, k, v through a short causal convolution per channel and silu; q, k unit vectors,
 //                 q times key_dim^-1/2; g = exp(-exp(A) softplus(xg + bg)), beta = sigmoid(xb):
 //                 decay = g, probe = g k, removal = beta k, write = beta k, read = q
+//   gated by channel   the same with one decay per head and key channel, g = exp(-exp(A_head) softplus(x + b))
 #include "common.h"
 
 #include "activations.h"
@@ -100,17 +101,18 @@ __device__ __forceinline__ float conv_at(const float* __restrict__ proj, size_t 
     return y;
 }
 
-// One wave per (token, head).  proj [T, C + nv + 2 heads]: q | k | v | gate | beta | rate.
-template <int KT>
+// One wave per (token, head).  proj [T, cols]: q | k | v | ..., beta's inputs (a number a head) from beta_column on;
+// the decay's inputs are columns of rates [T, rate_cols] from rate_column on, a number a head, or, CHANNEL, a number
+// a head and key channel (and rate_bias has as many).
+template <int KT, bool CHANNEL>
 __global__ __launch_bounds__(kWave) void gated_delta_prepare_kernel(
-    const float* __restrict__ proj, int T, int heads, int kv_heads, int dk, int dv, int K,
-    const float* __restrict__ taps, const float* __restrict__ tails, const float* __restrict__ rate_log,
-    const float* __restrict__ rate_bias, float unit_eps, const int* __restrict__ tok_req,
+    const float* __restrict__ proj, size_t cols, int beta_column, const float* __restrict__ rates, size_t rate_cols,
+    int rate_column, int T, int heads, int kv_heads, int dk, int dv, int K, const float* __restrict__ taps,
+    const float* __restrict__ tails, const float* __restrict__ rate_log, const float* __restrict__ rate_bias, float unit_eps, const int* __restrict__ tok_req,
     const int* __restrict__ q_offsets, const int* __restrict__ slot_ids, float* __restrict__ coef,
     float* __restrict__ v_out) {
     const int t = blockIdx.x / heads, head = blockIdx.x % heads, lane = threadIdx.x;
     const int nk = kv_heads * dk, nv = heads * dv, C = 2 * nk + nv;
-    const size_t cols = (size_t)C + nv + 2 * heads;
     const int r = tok_req[t];
     const int local = t - q_offsets[r];
     const float* tail = tails + (size_t)slot_ids[r] * (K - 1) * C;
@@ -130,8 +132,11 @@ __global__ __launch_bounds__(kWave) void gated_delta_prepare_kernel(
     const float q_inv = 1.f / (sqrtf(wave_sum(qq) + unit_eps) * sqrtf((float)dk));
     const float k_inv = 1.f / sqrtf(wave_sum(kk) + unit_eps);
     const float* row = proj + (size_t)t * cols;
-    const float beta = sigmoid(row[(size_t)C + nv + head]);
-    const float g = expf(-expf(rate_log[head]) * softplus_f(row[(size_t)C + nv + heads + head] + rate_bias[head]));
+    const float beta = sigmoid(row[beta_column + head]);
+    const float* rate = rates + (size_t)t * rate_cols + rate_column + (CHANNEL ? head * dk : head);
+    const float* bias = rate_bias + (CHANNEL ? head * dk : head);
+    const float speed = -expf(rate_log[head]);
+    float g = CHANNEL ? 0.f : expf(speed * softplus_f(rate[0] + bias[0]));
     const size_t plane = (size_t)T * heads * dk;
 #pragma unroll
     for (int e = 0; e < DELTA_PER_LANE; ++e) {
@@ -139,6 +144,7 @@ __global__ __launch_bounds__(kWave) void gated_delta_prepare_kernel(
         if (i >= dk) continue;
         const size_t at = ((size_t)t * heads + head) * dk + i;
         const float key = k[e] * k_inv;
+        if constexpr (CHANNEL) g = expf(speed * softplus_f(rate[i] + bias[i]));
         coef[at] = g;
         coef[plane + at] = g * key;
         coef[2 * plane + at] = beta * key;
@@ -448,23 +454,32 @@ LC_API int lc_general_delta_prepare(const float* proj, int T, int heads, int dim
     return 0;
 }
 
-LC_API int lc_gated_delta_prepare(const float* proj, int T, int heads, int kv_heads, int dk, int dv, int K,
-                                  const float* taps, const float* tails, int tail_slots, const float* rate_log,
-                                  const float* rate_bias, float unit_eps, const int* tok_req, const int* q_offsets,
-                                  const int* slot_ids, float* coef, float* v_out, hipStream_t stream) {
+static int gated_delta_prepare(bool by_channel, const float* proj, int cols, int beta_column, const float* rates,
+                               int rate_cols, int rate_column, int T, int heads, int kv_heads, int dk, int dv, int K,
+                               const float* taps, const float* tails, int tail_slots, const float* rate_log,
+                               const float* rate_bias, float unit_eps, const int* tok_req, const int* q_offsets,
+                               const int* slot_ids, float* coef, float* v_out, hipStream_t stream) {
     LC_CHECK(T >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dk > 0 && dv > 0,
              "gated_delta_prepare: bad sizes");
     LC_CHECK(dk <= DELTA_MAX_KEY, "gated_delta_prepare: heads of %d key channels are above %d", dk, DELTA_MAX_KEY);
     LC_CHECK(K >= 1 && K <= CONV_MAX_TAPS, "gated_delta_prepare: %d taps are outside 1..%d", K, CONV_MAX_TAPS);
+    LC_CHECK(beta_column >= 2 * kv_heads * dk + heads * dv && beta_column + heads <= cols && rate_column >= 0 &&
+                 rate_column + heads * (by_channel ? dk : 1) <= rate_cols,
+             "gated_delta_prepare: the gates' columns are outside their rows");
     if (T == 0) return 0;
-    LC_CHECK(proj && taps && rate_log && rate_bias && tok_req && q_offsets && slot_ids && coef && v_out &&
+    LC_CHECK(proj && rates && taps && rate_log && rate_bias && tok_req && q_offsets && slot_ids && coef && v_out &&
                  (tails || K == 1) && tail_slots >= 0,
              "gated_delta_prepare: null pointer");
     LC_CHECK((long long)T * heads < (1ll << 31), "gated_delta_prepare: too many heads");
-#define LC_PREPARE(KT)                                                                                              \
-    gated_delta_prepare_kernel<KT><<<T * heads, kWave, 0, stream>>>(proj, T, heads, kv_heads, dk, dv, K, taps, tails, \
-                                                                    rate_log, rate_bias, unit_eps, tok_req, q_offsets, \
-                                                                    slot_ids, coef, v_out)
+#define LC_PREPARE_AS(KT, CHANNEL)                                                                                \
+    gated_delta_prepare_kernel<KT, CHANNEL><<<T * heads, kWave, 0, stream>>>(                                       \
+        proj, (size_t)cols, beta_column, rates, (size_t)rate_cols, rate_column, T, heads, kv_heads, dk, dv, K, taps, \
+        tails, rate_log, rate_bias, unit_eps, tok_req, q_offsets, slot_ids, coef, v_out)
+#define LC_PREPARE(KT)                          \
+    do {                                        \
+        if (by_channel) LC_PREPARE_AS(KT, true); \
+        else LC_PREPARE_AS(KT, false);          \
+    } while (0)
     switch (K) {
         case 1: LC_PREPARE(1); break;
         case 2: LC_PREPARE(2); break;
@@ -477,8 +492,31 @@ LC_API int lc_gated_delta_prepare(const float* proj, int T, int heads, int kv_he
         default: LC_PREPARE(0); break;
     }
 #undef LC_PREPARE
+#undef LC_PREPARE_AS
     LC_LAUNCH_CHECK("gated_delta_prepare");
     return 0;
+}
+
+// proj [T, C + nv + 2 heads]: q | k | v | gate | beta | rate, the decay one number a head
+LC_API int lc_gated_delta_prepare(const float* proj, int T, int heads, int kv_heads, int dk, int dv, int K,
+                                  const float* taps, const float* tails, int tail_slots, const float* rate_log,
+                                  const float* rate_bias, float unit_eps, const int* tok_req, const int* q_offsets,
+                                  const int* slot_ids, float* coef, float* v_out, hipStream_t stream) {
+    const int C = 2 * kv_heads * dk + heads * dv, beta = C + heads * dv, cols = beta + 2 * heads;
+    return gated_delta_prepare(false, proj, cols, beta, proj, cols, beta + heads, T, heads, kv_heads, dk, dv, K, taps, tails,
+                               tail_slots, rate_log, rate_bias, unit_eps, tok_req, q_offsets, slot_ids, coef, v_out, stream);
+}
+
+// proj [T, cols]: q | k | v | ..., beta from beta_column on; rates [T, rate_cols]: the decay's inputs, heads x dk numbers
+// from rate_column on; rate_log [heads], rate_bias [heads dk]
+LC_API int lc_channel_delta_prepare(const float* proj, int cols, int beta_column, const float* rates, int rate_cols,
+                                    int rate_column, int T, int heads, int kv_heads, int dk, int dv, int K,
+                                    const float* taps, const float* tails, int tail_slots, const float* rate_log,
+                                    const float* rate_bias, float unit_eps, const int* tok_req, const int* q_offsets,
+                                    const int* slot_ids, float* coef, float* v_out, hipStream_t stream) {
+    return gated_delta_prepare(true, proj, cols, beta_column, rates, rate_cols, rate_column, T, heads, kv_heads, dk, dv, K,
+                               taps, tails, tail_slots, rate_log, rate_bias, unit_eps, tok_req, q_offsets, slot_ids, coef,
+                               v_out, stream);
 }
 
 LC_API int lc_conv_tail_update(const float* proj, int cols, int T, float* tails, int tail_slots, int C, int K,

@@ -372,7 +372,7 @@ LC_API int lc_gemm_grouped(const void* x, int x_dt, long long ldx, long long x_g
     LC_CHECK((row_start == nullptr) == (tile_start == nullptr), "grouped product: the lists come together");
     LC_CHECK(row_start || gather == nullptr, "grouped product: a gather list needs the rows' lists");
     LC_CHECK(!row_start || max_tiles > 0, "grouped product: no room for tiles");
-    LC_CHECK(epilogue >= ACT_NONE && epilogue <= ACT_SIGMOID_GROUP_GATE, "grouped product: unknown epilogue %d", epilogue);
+    LC_CHECK((epilogue >= ACT_NONE && epilogue <= ACT_SIGMOID_GROUP_GATE) || epilogue == ACT_GELU_ERF, "grouped product: unknown epilogue %d", epilogue);
     LC_CHECK((epilogue != ACT_SIGMOID_GATE && epilogue != ACT_SIGMOID_GROUP_GATE) || gate, "grouped product: no gates");
     LC_CHECK(tile_rows == 16 || tile_rows == 64 || tile_rows == 128, "grouped product: tiles of %d rows", tile_rows);
     LC_CHECK(G <= 65535 && (row_start ? max_tiles : (M + 15) / 16) <= 65535, "grouped product: too many tiles");

@@ -3,7 +3,8 @@
 //   q = silu(W_q h), k = silu(W_k h), v = silu(W_v h);   S <- decay S + k v^T;   o = S^T q
 // This file turns a step's float32 projections into the inputs of the framework's recurrence kernel
 // without its removal term (S <- diag(decay) S + write v^T, o = S^T read: three vectors a token), of
-// which lightning attention is the case decay = one number per head, write = k, read = q.
+// which lightning attention is the case decay = one number per head, write = k, read = q.  Gated linear attention is the
+// case of a decay per token and key channel, sigmoid(z)^power, with q scaled and no activations.
 #include "common.h"
 
 namespace lc {
@@ -28,6 +29,31 @@ __global__ void lightning_prepare_kernel(const float* __restrict__ proj, int col
             coef[2 * plane + at] = silu_f(row[c]);
         } else {
             v_out[(size_t)t * nv + (c - nk)] = silu_f(row[2 * nk + (c - nk)]);
+        }
+    }
+}
+
+// proj [T, cols]: q | k (heads x dk each) | v (heads x dv) | ...; z: columns z_column .. + heads dk of rates; the decay is
+// sigmoid(z + bias)^power = exp(-power ln(1 + e^-(z + bias)))
+__global__ void gated_linear_prepare_kernel(const float* __restrict__ proj, int cols, const float* __restrict__ rates,
+                                            int rate_cols, int z_column, const float* __restrict__ bias, float power,
+                                            float q_scale, int T, int heads, int dk, int dv, float* __restrict__ coef,
+                                            float* __restrict__ v_out) {
+    const int nk = heads * dk, nv = heads * dv;
+    const size_t plane = (size_t)T * nk;
+    const size_t total = (size_t)T * (nk + nv);
+    for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
+         idx += (size_t)gridDim.x * blockDim.x) {
+        const int t = (int)(idx / (nk + nv)), c = (int)(idx % (nk + nv));
+        const float* row = proj + (size_t)t * cols;
+        if (c < nk) {
+            const size_t at = (size_t)t * nk + c;
+            const float z = rates[(size_t)t * rate_cols + z_column + c] + bias[c];
+            coef[at] = expf(-power * (fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z)))));
+            coef[plane + at] = row[nk + c];
+            coef[2 * plane + at] = row[c] * q_scale;
+        } else {
+            v_out[(size_t)t * nv + (c - nk)] = row[2 * nk + (c - nk)];
         }
     }
 }
@@ -67,6 +93,22 @@ LC_API int lc_lightning_readout(const float* o, const float* gates, int gate_col
     else
         LC_CHECK(false, "lightning readout: unknown dtype %d", dt);
     LC_LAUNCH_CHECK("lightning_readout");
+    return 0;
+}
+
+LC_API int lc_gated_linear_prepare(const float* proj, int cols, const float* rates, int rate_cols, int z_column,
+                                   const float* bias, float power, float q_scale, int T, int heads, int dk, int dv,
+                                   float* coef, float* v_out, hipStream_t stream) {
+    LC_CHECK(T >= 0 && heads > 0 && dk > 0 && dv > 0 && cols >= heads * (2 * dk + dv) && z_column >= 0 &&
+                 z_column + heads * dk <= rate_cols,
+             "gated linear prepare: bad sizes");
+    if (T == 0) return 0;
+    LC_CHECK(proj && rates && bias && coef && v_out, "gated linear prepare: null pointer");
+    const size_t total = (size_t)T * heads * (dk + dv);
+    const int blocks = (int)((total + 255) / 256 < 8192 ? (total + 255) / 256 : 8192);
+    gated_linear_prepare_kernel<<<blocks, 256, 0, stream>>>(proj, cols, rates, rate_cols, z_column, bias, power, q_scale, T,
+                                                            heads, dk, dv, coef, v_out);
+    LC_LAUNCH_CHECK("gated_linear_prepare");
     return 0;
 }
 

@@ -1,11 +1,12 @@
 // Attention over a paged cache with the things the framework's other attention kernels do not know:
 // keys and values of different head counts and sizes, several score maps per head over the same values
-// (differential attention), a mask of chunks, a bias that grows with the logarithm of the distance, and a
-// sink in the softmax's denominator.  Float32 arithmetic throughout; one workgroup per token and head.
+// (differential attention), masks of chunks or windows, kept first keys, a bias that grows with the logarithm of the
+// distance, scores held below a cap, and a sink in the softmax's denominator.  Float32 arithmetic throughout; one workgroup per token and head.
 //
 // With p the query's position, the visible keys are lo .. p, lo = max(p - p % chunk (chunk > 0),
-// p - window + 1 (window > 0), 0).  Per head h (kv head g = h / (heads / kv_heads)) and map m < maps:
+// p - window + 1 (window > 0), 0), and those of the first `keep` that lie before lo.  Per head h (kv head g = h / (heads / kv_heads)) and map m < maps:
 //   s_j = scale (q_(h,m) . k_(g,m),j) - r1_h ln(1 + r2_h (p - j))            (the bias where r1 is given)
+//   cap > 0: s_j <- cap tanh(s_j / cap)
 //   a_m = sum_j exp(s_j) v_g,j / (sum_j exp(s_j) + exp(sink_h))              (the sink where it is given)
 //   maps = 1: o = a_0;   maps = 2: o = a_0 - lambda a_1
 //   unit_out: o <- o / sqrt(mean(o^2) + eps) * out_scale;   gate: o <- o sigmoid(gate_(h, .))
@@ -13,7 +14,7 @@
 // kv_heads * dv, page] (the matrix-core kernel's operand wants a value entry's neighbouring keys side by side).
 // Position j of request r lies in page block_table[r][j / page] at place j % page.
 //
-// The keys are walked in tiles of 256 from lo on, with a running maximum and sum per map: the order of
+// The kept keys and those from lo on are walked as one list in tiles of 256, with a running maximum and sum per map: the order of
 // every addition is a function of the query's position alone, so a token's result has the same bits in
 // every batch and for every cut of its prompt.
 //
@@ -53,7 +54,7 @@ __global__ __launch_bounds__(MA_THREADS) void masked_attention_kernel(
     const T* __restrict__ q, const T* __restrict__ k_cache, const T* __restrict__ v_cache,
     const int* __restrict__ tok_req, const int* __restrict__ positions, const int* __restrict__ block_table,
     int max_blocks, int page_size, int heads, int kv_heads, int d, int dv, int dv_pow2, float scale, int chunk,
-    int window, const float* __restrict__ r1, const float* __restrict__ r2, const float* __restrict__ sink,
+    int window, int keep, float cap, const float* __restrict__ r1, const float* __restrict__ r2, const float* __restrict__ sink,
     float lambda, int unit_out, float eps, float out_scale, const float* __restrict__ gate, int gate_stride,
     int gate_column, T* __restrict__ out) {
     __shared__ __align__(16) float qs[MAPS][MA_MAX];
@@ -78,18 +79,23 @@ __global__ __launch_bounds__(MA_THREADS) void masked_attention_kernel(
 #pragma unroll
     for (int m = 0; m < MAPS; ++m) { M[m] = -INFINITY; L[m] = 0.f; acc[m] = 0.f; }
     __syncthreads();
-    for (int c0 = lo; c0 <= p; c0 += MA_THREADS) {
-        const int count = min(MA_THREADS, p - c0 + 1);
+    // the visible keys as one list: the kept ones before lo, then lo .. p
+    const int kept = min(keep, lo), visible = kept + p - lo + 1;
+    auto key_at = [&](int i) { return i < kept ? i : lo + (i - kept); };
+    for (int c0 = 0; c0 < visible; c0 += MA_THREADS) {
+        const int count = min(MA_THREADS, visible - c0);
         float s[MAPS];
 #pragma unroll
         for (int m = 0; m < MAPS; ++m) s[m] = -INFINITY;
         if (tid < count) {
-            const int j = c0 + tid;
+            const int j = key_at(c0 + tid);
             const size_t row = (size_t)table[j / page_size] * page_size + j % page_size;
             const float far = r1 ? bias1 * log1pf(bias2 * (float)(p - j)) : 0.f;
 #pragma unroll
-            for (int m = 0; m < MAPS; ++m)
+            for (int m = 0; m < MAPS; ++m) {
                 s[m] = dot_row(qs[m], k_cache + row * k_row + ((size_t)g * MAPS + m) * d, d) - far;
+                if (cap > 0.f) s[m] = cap * tanhf(s[m] / cap);
+            }
         }
 #pragma unroll
         for (int m = 0; m < MAPS; ++m) {
@@ -104,7 +110,7 @@ __global__ __launch_bounds__(MA_THREADS) void masked_attention_kernel(
         __syncthreads();
         if (active)
             for (int jj = grp; jj < count; jj += groups) {
-                const int j = c0 + jj;
+                const int j = key_at(c0 + jj);
                 const float v = to_f32(v_cache[((size_t)table[j / page_size] * v_row + (size_t)g * dv + dim) * page_size
                                                + j % page_size]);
 #pragma unroll
@@ -278,7 +284,7 @@ using namespace lc;
 
 LC_API int lc_masked_attention(const void* q, const void* k_cache, const void* v_cache, int dt, const int* tok_req,
                                const int* positions, const int* block_table, int max_blocks, int page_size, int T,
-                               int heads, int kv_heads, int maps, int d, int dv, float scale, int chunk, int window,
+                               int heads, int kv_heads, int maps, int d, int dv, float scale, int chunk, int window, int keep, float cap,
                                const float* r1, const float* r2, const float* sink, float lambda, int unit_out,
                                float eps, float out_scale, const float* gate, int gate_stride, int gate_column,
                                void* out, hipStream_t stream) {
@@ -290,7 +296,7 @@ LC_API int lc_masked_attention(const void* q, const void* k_cache, const void* v
     LC_CHECK(maps == 1 || maps == 2, "masked attention: %d score maps a head (1 or 2)", maps);
     LC_CHECK(d <= MA_MAX && dv <= MA_MAX, "masked attention: heads of %d/%d entries are above %d", d, dv, MA_MAX);
     LC_CHECK(heads <= 65535, "masked attention: too many heads (%d)", heads);
-    LC_CHECK(chunk >= 0 && window >= 0, "masked attention: bad mask");
+    LC_CHECK(chunk >= 0 && window >= 0 && keep >= 0 && cap >= 0.f, "masked attention: bad mask or cap");
     LC_CHECK(q && k_cache && v_cache && out && tok_req && positions && block_table, "masked attention: null pointer");
     LC_CHECK((r1 == nullptr) == (r2 == nullptr), "masked attention: the bias needs both of its vectors");
     LC_CHECK(!gate || (gate_column >= 0 && gate_column + heads * dv <= gate_stride), "masked attention: bad gate columns");
@@ -300,7 +306,7 @@ LC_API int lc_masked_attention(const void* q, const void* k_cache, const void* v
 #define LC_MA(TT, MAPS)                                                                                              \
     masked_attention_kernel<TT, MAPS><<<grid, MA_THREADS, 0, stream>>>(                                               \
         (const TT*)q, (const TT*)k_cache, (const TT*)v_cache, tok_req, positions, block_table, max_blocks, page_size, \
-        heads, kv_heads, d, dv, dv_pow2, scale, chunk, window, r1, r2, sink, lambda, unit_out, eps, out_scale, gate,  \
+        heads, kv_heads, d, dv, dv_pow2, scale, chunk, window, keep, cap, r1, r2, sink, lambda, unit_out, eps, out_scale, gate,  \
         gate_stride, gate_column, (TT*)out)
     if (dt == DT_F32) { if (maps == 1) LC_MA(float, 1); else LC_MA(float, 2); }
     else if (dt == DT_BF16) { if (maps == 1) LC_MA(bf16, 1); else LC_MA(bf16, 2); }

@@ -38,7 +38,8 @@ struct MaskedArgs {
     const int* block_table;
     int max_blocks, page_size, heads, kv_heads, d, dv;
     float scale;
-    int chunk, window;
+    int chunk, window, keep;
+    float cap;          // scores become cap tanh(score / cap) where it is positive
     const float* r1;
     const float* r2;
     const float* sink;
@@ -58,6 +59,12 @@ struct MaskedArgs {
 template <int DVB> constexpr int share_floats() { return DVB * 4 + 2; }
 
 __device__ __forceinline__ short bits_of(__bf16 v) { return __builtin_bit_cast(short, v); }
+
+// s held below cap: cap tanh(s / cap) = cap (1 - 2 / (1 + e^(2 s / cap))); the ends saturate to +-cap
+__device__ __forceinline__ float held(float s, float cap) {
+    if (cap <= 0.f) return s;
+    return cap - 2.f * cap / (1.f + __expf(2.f * s / cap));
+}
 
 // over the four lanes that hold one query column (lane, lane ^ 16, lane ^ 32, lane ^ 48)
 __device__ __forceinline__ float column_max4(float v) {
@@ -96,14 +103,14 @@ __device__ __forceinline__ void block_step(ColumnState<DVB, MAPS>& st, const Mas
         if (all_seen) {             // every column of the wave sees the whole block: nothing to mask
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
-                s[v] = fmaf(s[v], a.scale, -far[v]);
+                s[v] = held(fmaf(s[v], a.scale, -far[v]), a.cap);
                 mx = fmaxf(mx, s[v]);
             }
         } else {
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
                 const int j = j0 + v;
-                s[v] = (j >= lo && j <= pos) ? fmaf(s[v], a.scale, -far[v]) : -INFINITY;
+                s[v] = ((j >= lo || j < a.keep) && j <= pos) ? held(fmaf(s[v], a.scale, -far[v]), a.cap) : -INFINITY;
                 mx = fmaxf(mx, s[v]);
             }
         }
@@ -145,6 +152,17 @@ __device__ __forceinline__ void block_step(ColumnState<DVB, MAPS>& st, const Mas
     }
 }
 
+// The blocks of 16 keys a tile walks: those that hold kept keys and lie before the first visible block, then the blocks
+// first .. last.
+struct BlockList {
+    int kept, first, count;
+    __device__ __forceinline__ int block(int i) const { return i < kept ? i : first + (i - kept); }
+};
+__device__ __forceinline__ BlockList block_list(int keep, int first, int last) {
+    const int kept = min((keep + 15) / 16, first);
+    return {kept, first, kept + last - first + 1};
+}
+
 template <int DSTEPS, int MAPS>
 __device__ __forceinline__ void load_queries(bf16x8 (&bq)[MAPS][DSTEPS], const MaskedArgs& a, int tok, int head, int pos,
                                              int lane) {
@@ -173,12 +191,13 @@ __device__ __forceinline__ void clear_state(ColumnState<DVB, MAPS>& st) {
 }
 
 // The lane's column: token row `tok`, head `head`, position `pos` (-1: no such column), first visible key `lo`.
-// Blocks first, first + stride, ... <= last of 16 keys each.  Keys seen_from .. seen_to are seen by every column of
+// The blocks of 16 keys to walk are a list, the kept ones in front (BlockList); the lane's wave takes the list's places
+// at, at + stride, ....  Keys seen_from .. seen_to are seen by every column of
 // the tile (a block inside them needs no mask).
 template <int DSTEPS, int DVB, int MAPS>
 __device__ __forceinline__ void attend_blocks(ColumnState<DVB, MAPS>& st, const MaskedArgs& a, int g, int tok, int head,
-                                              int pos, int lo, const int* __restrict__ table, int first, int last,
-                                              int stride, int seen_from, int seen_to, int lane) {
+                                              int pos, int lo, const int* __restrict__ table, const BlockList& blocks,
+                                              int at, int stride, int seen_from, int seen_to, int lane) {
     const int quad = lane >> 4, col = lane & 15;
     const size_t k_row = (size_t)a.kv_heads * MAPS * a.d;
     bf16x8 bq[MAPS][DSTEPS];
@@ -214,19 +233,19 @@ __device__ __forceinline__ void attend_blocks(ColumnState<DVB, MAPS>& st, const 
     constexpr bool VALUES_AHEAD = DSTEPS * MAPS * 4 + DVB * MAPS * 4 + DVB * 4 <= 120;
     bf16x8 ka[MAPS][DSTEPS], kn[MAPS][DSTEPS];
     short4v va[DVB], vn[DVB];
-    if (first <= last) {
-        load_keys(ka, first);
-        if constexpr (VALUES_AHEAD) load_values(va, first);
+    if (at < blocks.count) {
+        load_keys(ka, blocks.block(at));
+        if constexpr (VALUES_AHEAD) load_values(va, blocks.block(at));
     }
-    for (int b = first; b <= last; b += stride) {
-        const int key0 = b * 16;
+    for (int i = at; i < blocks.count; i += stride) {
+        const int b = blocks.block(i), key0 = b * 16;
         if constexpr (!VALUES_AHEAD) load_values(va, b);
-        if (b + stride <= last) {           // on their way while this block is worked on
-            load_keys(kn, b + stride);
-            if constexpr (VALUES_AHEAD) load_values(vn, b + stride);
+        if (i + stride < blocks.count) {            // on their way while this block is worked on
+            load_keys(kn, blocks.block(i + stride));
+            if constexpr (VALUES_AHEAD) load_values(vn, blocks.block(i + stride));
         }
         block_step<DSTEPS, DVB, MAPS>(st, a, bq, ka, va, key0, pos, lo, bias1, bias2,
-                                      key0 >= seen_from && key0 + 15 <= seen_to, lane);
+                                      (key0 >= seen_from || key0 + 15 < a.keep) && key0 + 15 <= seen_to, lane);
 #pragma unroll
         for (int m = 0; m < MAPS; ++m)
 #pragma unroll
@@ -309,8 +328,8 @@ __global__ __launch_bounds__(MB_THREADS) void masked_attention_bf16_kernel(Maske
         while (places < group && places < MB_WAVES) places *= 2;
     const int splits = MB_WAVES / places;
     const int place = wave % places, split = wave / places;
-    // the blocks from the first token's first key to the last token
-    const int first = first_key(p0) / 16, last = (p0 + n - 1) / 16;
+    // the kept blocks, then those from the first token's first key to the last token
+    const BlockList blocks = block_list(a.keep, first_key(p0) / 16, (p0 + n - 1) / 16);
     // what every token of the tile sees: from the last token's first key to the first token (a column without a token
     // or head computes on zeros there and is never written)
     const int seen_from = first_key(p0 + n - 1), seen_to = p0;
@@ -326,7 +345,7 @@ __global__ __launch_bounds__(MB_THREADS) void masked_attention_bf16_kernel(Maske
         const int lo = on ? first_key(pos) : 0;
         const bool wave_on = lone || h0 + place < group;
         if (wave_on)
-            attend_blocks<DSTEPS, DVB, MAPS>(st, a, g, tok, head, pos, lo, table, first + z * splits + split, last,
+            attend_blocks<DSTEPS, DVB, MAPS>(st, a, g, tok, head, pos, lo, table, blocks, z * splits + split,
                                              splits * zsplits, seen_from, seen_to, lane);
         if (splits > 1) {
 #pragma unroll
@@ -409,9 +428,9 @@ __global__ __launch_bounds__(MB_THREADS) void masked_attention_bf16_staged_kerne
     while (places < group && places < MB_WAVES) places *= 2;
     const int splits = min(MB_WAVES / places, MB_STAGE_BLOCKS);      // waves that share a head's keys
     const int place = wave % places, split = wave / places;
-    const int first = first_key(p0) / 16, last = (p0 + n - 1) / 16;
+    const BlockList blocks = block_list(a.keep, first_key(p0) / 16, (p0 + n - 1) / 16);
     const int stage_blocks = splits * a.wave_blocks;
-    const int stages = (last - first + stage_blocks) / stage_blocks;
+    const int stages = (blocks.count + stage_blocks - 1) / stage_blocks;
     const int seen_from = first_key(p0 + n - 1);        // every token of the tile sees the keys from here to p0
     const bool full_sizes = a.d == DSTEPS * 32 && a.dv == DVB * 16;
     const int d_all = MAPS * a.d;                               // a key row's entries of this kv head
@@ -425,12 +444,12 @@ __global__ __launch_bounds__(MB_THREADS) void masked_attention_bf16_staged_kerne
     // block of values: no division by a size that only the launch knows); places beyond the real sizes stay empty.
     constexpr int KP = DSTEPS * 4 * MAPS, VP = DVB * 32, MAX_BLOCKS = 2 * MB_STAGE_BLOCKS;
     auto fetch = [&](int stage) {
-        const int b0 = first + stage * stage_blocks;
+        const int b0 = stage * stage_blocks;
         int page_of[MAX_BLOCKS], within_of[MAX_BLOCKS];         // the same for all threads
 #pragma unroll
         for (int blk = 0; blk < MAX_BLOCKS; ++blk) {
-            const int key0 = (b0 + blk) * 16;
-            const bool there = blk < stage_blocks && b0 + blk <= last;
+            const int key0 = blocks.block(b0 + blk) * 16;
+            const bool there = blk < stage_blocks && b0 + blk < blocks.count;
             page_of[blk] = there ? table[key0 / a.page_size] : -1;
             within_of[blk] = key0 % a.page_size;
         }
@@ -496,8 +515,9 @@ __global__ __launch_bounds__(MB_THREADS) void masked_attention_bf16_staged_kerne
         for (int stage = 0; stage < stages; ++stage) {
             if (stage + 1 < stages) fetch(stage + 1);       // on its way while this stage is worked on
             for (int j = 0; j < a.wave_blocks; ++j) {
-                const int blk = j * splits + split, b = first + stage * stage_blocks + blk;
-                if (!wave_on || b > last) continue;
+                const int blk = j * splits + split, place_of = stage * stage_blocks + blk;
+                if (!wave_on || place_of >= blocks.count) continue;
+                const int b = blocks.block(place_of);
                 bf16x8 ka[MAPS][DSTEPS];
                 short4v va[DVB];
                 const unsigned char* krow = staged + (blk * 16 + col) * k_pitch + quad * 16;
@@ -527,7 +547,7 @@ __global__ __launch_bounds__(MB_THREADS) void masked_attention_bf16_staged_kerne
                     }
                 }
                 block_step<DSTEPS, DVB, MAPS>(st, a, bq, ka, va, b * 16, pos, lo, bias1, bias2,
-                                              b * 16 >= seen_from && b * 16 + 15 <= p0, lane);
+                                              (b * 16 >= seen_from || b * 16 + 15 < a.keep) && b * 16 + 15 <= p0, lane);
             }
             __syncthreads();                    // every wave has read the stage
             if (stage + 1 < stages) store();
@@ -638,7 +658,7 @@ LC_API long long lc_masked_attention_bf16_workspace(int num_tiles, int heads, in
 LC_API int lc_masked_attention_bf16(const void* q, const void* k_cache, const void* v_cache, const int* tiles,
                                     int num_tiles, const int* block_table, int max_blocks, int page_size, int heads,
                                     int kv_heads, int maps, int d, int dv, float scale, int chunk, int window,
-                                    const float* r1, const float* r2, const float* sink, float lambda, int unit_out,
+                                    int keep, float cap, const float* r1, const float* r2, const float* sink, float lambda, int unit_out,
                                     float eps, float out_scale, const float* gate, int gate_stride, int gate_column,
                                     void* out, float* shares, int zsplits, int any_portion, int any_lone,
                                     hipStream_t stream) {
@@ -651,8 +671,9 @@ LC_API int lc_masked_attention_bf16(const void* q, const void* k_cache, const vo
     LC_CHECK(q && k_cache && v_cache && tiles && block_table && out, "masked attention: null pointer");
     LC_CHECK((r1 == nullptr) == (r2 == nullptr), "masked attention: the bias needs both of its vectors");
     LC_CHECK(kv_heads <= 65535, "masked attention: too many kv heads");
+    LC_CHECK(chunk >= 0 && window >= 0 && keep >= 0 && cap >= 0.f, "masked attention: bad mask or cap");
     MaskedArgs a{(const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, tiles, block_table, max_blocks, page_size,
-                 heads, kv_heads, d, dv, scale, chunk, window, r1, r2, sink, lambda, unit_out, eps, out_scale, gate,
+                 heads, kv_heads, d, dv, scale, chunk, window, keep, cap, r1, r2, sink, lambda, unit_out, eps, out_scale, gate,
                  gate_stride, gate_column, (bf16*)out, shares, zsplits, 0, 1};
     // tiles of several tokens go through the kernel that stages keys and values in LDS where a stage fits a thread's
     // two pieces of each kind

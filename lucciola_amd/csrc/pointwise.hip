@@ -4,6 +4,7 @@
 // All arithmetic is float32; only loads and stores have the tensors' types.
 //   dynamic tanh   y = tanh(alpha v) w + b,  v = h (+ delta)
 //   gelu (tanh)    0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
+//   gelu (erf)     0.5 z (1 + erf(z / sqrt(2)))
 //   relu squared   max(z, 0)^2
 //   xIELU          z > 0: a z^2 + z/2;  z <= 0: b (e^z - 1 - z) + z/2
 // and the token shift: what a mixer reads of token t becomes x_t + (x_(t-1) - x_t) mix, the row before
@@ -188,9 +189,9 @@ LC_API int lc_stream_add(float* h, const void* delta, int dt, const float* more,
     return 0;
 }
 
-// kind: 1 gelu (tanh form), 2 relu squared, 5 xIELU with its two numbers (a, b); in place
+// kind: 1 gelu (tanh form), 6 gelu (with the error function), 2 relu squared, 5 xIELU with its two numbers (a, b); in place
 LC_API int lc_activation(void* x, int dt, int kind, float a, float b, long long total, hipStream_t stream) {
-    LC_CHECK(total >= 0 && (kind == ACT_GELU_TANH || kind == ACT_RELU_SQUARED || kind == ACT_XIELU),
+    LC_CHECK(total >= 0 && (kind == ACT_GELU_TANH || kind == ACT_GELU_ERF || kind == ACT_RELU_SQUARED || kind == ACT_XIELU),
              "activation: bad arguments");
     if (total == 0) return 0;
     LC_CHECK(x, "activation: null pointer");

@@ -11,7 +11,7 @@ import ctypes
 import heapq
 import threading
 from dataclasses import dataclass, replace
-from typing import Optional
+from typing import Optional, Tuple
 
 import numpy as np
 import torch
@@ -104,11 +104,11 @@ _SIGNATURES = {
     "lc_moe_route_logits": "pipiiippp",
     "lc_moe_combine_shared": "pppiiipipiipip",
     "lc_gated_activation_weighted": "ppippiiip",
-    "lc_masked_attention": "pppi" + "ppp" + "ii" + "i" + "iiiii" + "f" + "ii" + "ppp" + "f" + "i" + "ff" + "pii" + "pp",
+    "lc_masked_attention": "pppi" + "ppp" + "ii" + "i" + "iiiii" + "f" + "iiif" + "ppp" + "f" + "i" + "ff" + "pii" + "pp",
     "lc_attention_prepare": "p" + "iiiiiii" + "pip" + "ppp" + "pip" + "if" + "ppp" + "i" + "pip",
     "lc_attention_prepare_pairs": "i",
     "lc_masked_attention_bf16_supported": "iiii",
-    "lc_masked_attention_bf16": "ppp" + "pi" + "pii" + "iiiii" + "f" + "ii" + "ppp" + "f" + "i" + "ff" + "pii" + "ppiiip",
+    "lc_masked_attention_bf16": "ppp" + "pi" + "pii" + "iiiii" + "f" + "iiif" + "ppp" + "f" + "i" + "ff" + "pii" + "ppiiip",
     "lc_masked_attention_bf16_staged": "i",
     "lc_masked_attention_bf16_workspace": "iiiiii",
     "lc_state_space_prepare": "piiiiii" + "ppi" + "ppp" + "ppp" + "pp" + "p",
@@ -118,6 +118,10 @@ _SIGNATURES = {
     "lc_attention_rows": "piiiiiii" + "pppf" + "piip" + "pfp" + "pppipi" + "p",
     "lc_mlstm_prepare": "piiippf" + "pippi" + "iiiifi" + "ppp" + "p",
     "lc_mlstm_readout": "ppfpiipfiiipip",
+    "lc_attention_heads": "piiiiiii" + "i" + "pppf" + "piip" + "ff" + "pppipi" + "p",
+    "lc_channel_delta_prepare": "piipii" + "iiiiii" + "ppi" + "ppf" + "ppp" + "pp" + "p",
+    "lc_gated_linear_prepare": "pipiipff" + "iiii" + "pp" + "p",
+    "lc_stream_norms": "ppiiii" + 3 * "piifpp" + "ppfppi" + "p",
 }
 
 
@@ -330,9 +334,111 @@ class ProductShares:
         return out
 
 
+@dataclass
+class RoutedRows:
+    """A mixture of experts' output that has not been put together yet: token t's is the sum over its choices of
+    the routing's weight times the row of float32 ``y`` [T top, n] that the choice's place names."""
+
+    y: torch.Tensor
+    routing: "Routing"
+    out_dtype: torch.dtype
+
+    def value(self) -> torch.Tensor:
+        return moe_combine(self.y, self.routing, self.out_dtype)
+
+
+@dataclass
+class SummedBranches:
+    """Several branches' outputs that wait together to be added to the residual stream, ``scale`` times ``output`` each
+    (a tensor, a PendingProduct or RoutedRows): :func:`stream_norms` and :func:`rmsnorm` take them as the stream's
+    pending addition; anyone else gets the float32 sum from ``value()``."""
+
+    branches: Tuple[Tuple[object, float], ...]
+
+    def value(self) -> torch.Tensor:
+        total = None
+        for output, scale in self.branches:
+            x = value(output)
+            if total is None:
+                total, first = x, scale
+            else:
+                total, first = scaled_sum(total, first, x, scale), 1.0
+        return scaled_sum(total, first, total, 0.0) if first != 1.0 or total.dtype != torch.float32 else total
+
+
+def summed(*parts) -> SummedBranches:
+    """``(output, scale)`` pairs as one pending addition; an output that is itself a sum is taken apart."""
+    flat = []
+    for output, scale in parts:
+        if isinstance(output, SummedBranches):
+            flat.extend((o, s * scale) for o, s in output.branches)
+        else:
+            flat.append((output, float(scale)))
+    return SummedBranches(tuple(flat))
+
+
+STREAM_ADDENDS = 3      # branches that one norm kernel takes in
+
+
+def stream_norms(h: torch.Tensor, delta, weights, eps: float, out_dtype: torch.dtype,
+                 rows: Optional[torch.Tensor] = None) -> Tuple[torch.Tensor, ...]:
+    """The float32 residual stream ``h`` [T, n] with the pending ``delta`` (None, a tensor, a PendingProduct, RoutedRows
+    or SummedBranches of up to three of them) added, divided by its root mean square (``eps`` inside the root) and
+    multiplied by each of the one or two ``weights`` float32 [n].  Without ``rows`` h becomes the sum; with ``rows``
+    (int32 [R]) only those rows are normed and h stays as it is.  -> a tensor per weight."""
+    _need(h, "stream_norms h", torch.float32, 2)
+    T, n = h.shape
+    if not 1 <= len(weights) <= 2:
+        raise KernelError(f"stream_norms: {len(weights)} weights (1 or 2)")
+    for w in weights:
+        _need(w, "stream_norms weight", torch.float32, 1)
+        if w.shape[0] != n:
+            raise KernelError(f"stream_norms: a weight of {w.shape[0]} entries for rows of {n}")
+    if rows is not None:
+        _need(rows, "stream_norms rows", torch.int32, 1)
+    branches = () if delta is None else delta.branches if isinstance(delta, SummedBranches) else ((delta, 1.0),)
+    if len(branches) > STREAM_ADDENDS:
+        raise KernelError(f"stream_norms: {len(branches)} branches are above the kernel's {STREAM_ADDENDS}")
+    R = T if rows is None else rows.shape[0]
+    args, held = [], []
+    for output, scale in branches:
+        kind, count, by, places = 0, 0, None, None
+        if isinstance(output, RoutedRows):
+            t, routing = output.y, output.routing
+            _need(t, "stream_norms routed rows", torch.float32, 2)
+            kind, count, by, places = 4, routing.ids.shape[1], routing.weights, routing.entry_row
+            if tuple(t.shape) != (T * count, n):
+                raise KernelError(f"stream_norms: routed rows {tuple(t.shape)} for {T} tokens of {count} choices")
+        else:
+            t = None
+            if isinstance(output, PendingProduct):
+                M, K = output.x.shape
+                count = library().lc_gemm_bf16_shares(M, n, K) if (output.w.shape[0] == n and M == T) else 0
+                if count:       # the product is cut along K anyway: its shares are summed in the norm kernel
+                    t, kind = torch.empty((count, T, n), dtype=torch.float32, device=h.device), 3
+                    _call("lc_gemm_bf16_partials", _ptr(output.x), _ptr(output.w), _ptr(t), _c_int(M), _c_int(n),
+                          _c_int(K), _stream())
+            if t is None:
+                t, count = value(output), 0
+                _need(t, "stream_norms branch", None, 2)
+                if tuple(t.shape) != (T, n) or t.dtype not in (torch.float32, torch.bfloat16):
+                    raise KernelError(f"stream_norms: a branch {tuple(t.shape)} of {t.dtype} for a stream {(T, n)}")
+                kind = 1 if t.dtype == torch.float32 else 2
+        held.append(t)
+        args += [_ptr(t), kind, count, float(scale), _ptr(by), _ptr(places)]
+    args += [None, 0, 0, 0.0, None, None] * (STREAM_ADDENDS - len(branches))
+    outs = tuple(torch.empty((R, n), dtype=out_dtype, device=h.device) for _ in weights)
+    if R:
+        second = len(weights) == 2
+        _call("lc_stream_norms", _ptr(h), _ptr(rows), R, T, n, 1 if rows is None and branches else 0, *args,
+              _ptr(weights[0]), _ptr(weights[1] if second else None), float(eps), _ptr(outs[0]),
+              _ptr(outs[1] if second else None), _dt(outs[0]), _stream())
+    return outs
+
+
 def value(t):
     """The tensor that ``t`` stands for (``t`` itself if it is one)."""
-    return t.value() if isinstance(t, (PendingProduct, ScaledRows, ProductShares, NormedBranch, BiasedBranch)) else t
+    return t.value() if isinstance(t, (PendingProduct, ScaledRows, ProductShares, NormedBranch, BiasedBranch, RoutedRows, SummedBranches)) else t
 
 
 def rmsnorm(h: torch.Tensor, delta, weight: torch.Tensor, eps: float,
@@ -344,6 +450,8 @@ def rmsnorm(h: torch.Tensor, delta, weight: torch.Tensor, eps: float,
     [R]): only those rows are normed (``h`` stays as it is) and the result is [R, n].
     ``scaled``: the caller also takes ScaledRows, and gets them where that saves a kernel.
     """
+    if isinstance(delta, SummedBranches):
+        return stream_norms(h, delta, (weight,), eps, out_dtype, rows=rows)[0]
     _need(h, "rmsnorm h", torch.float32, 2)
     _need(weight, "rmsnorm weight", torch.float32, 1)
     T, n = h.shape
@@ -958,9 +1066,9 @@ def swiglu(gu: torch.Tensor) -> torch.Tensor:
 
 
 # ------------------------------------------------------------------------------ other norms, other feed-forwards
-ACTIVATIONS = {"gelu_tanh": 1, "relu_squared": 2, "xielu": 5}     # xielu takes two numbers (``params``)
+ACTIVATIONS = {"gelu_tanh": 1, "relu_squared": 2, "xielu": 5, "gelu": 6}     # xielu takes two numbers (``params``)
 _EPILOGUE_GATE, _EPILOGUE_GROUP_GATE = 3, 4
-_EPILOGUES = {"gelu_tanh": 1, "relu_squared": 2}                    # what a grouped product can apply itself
+_EPILOGUES = {"gelu_tanh": 1, "relu_squared": 2, "gelu": 6}                    # what a grouped product can apply itself
 
 
 def dynamic_tanh(h: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Tensor, bias: torch.Tensor,
@@ -1675,6 +1783,47 @@ def gated_delta_prepare(proj: torch.Tensor, tail: torch.Tensor, taps: torch.Tens
     return coef, v
 
 
+def channel_delta_prepare(proj: torch.Tensor, beta_column: int, rates: torch.Tensor, rate_column: int,
+                          tail: Optional[torch.Tensor], taps: torch.Tensor, rate_log: torch.Tensor,
+                          rate_bias: torch.Tensor, heads: int, kv_heads: int, key_dim: int, value_dim: int,
+                          num_taps: int, unit_eps: float, tok_req: torch.Tensor, q_offsets: torch.Tensor,
+                          slot_ids: torch.Tensor):
+    """As :func:`gated_delta_prepare` with a decay per head and key channel: ``proj`` float32 [T, cols] holds q | k | v
+    in its first columns and beta's inputs from ``beta_column`` on; the decay's inputs are the heads key_dim columns of
+    float32 ``rates`` from ``rate_column`` on, g = exp(-exp(rate_log[head]) softplus(rate + rate_bias)) with
+    ``rate_bias`` [heads key_dim]."""
+    _need(proj, "channel_delta proj", torch.float32, 2)
+    _need(rates, "channel_delta rates", torch.float32, 2)
+    T = proj.shape[0]
+    nk = heads * key_dim
+    C = 2 * kv_heads * key_dim + heads * value_dim
+    if beta_column < C or beta_column + heads > proj.shape[1] or rates.shape[0] != T or rate_column < 0 \
+            or rate_column + nk > rates.shape[1]:
+        raise KernelError("channel_delta_prepare: the projections do not fit the heads")
+    _need(taps, "conv taps", torch.float32, 2)
+    if tuple(taps.shape) != (C, num_taps):
+        raise KernelError("channel_delta_prepare: the taps do not fit the channels")
+    if num_taps > 1:
+        _need(tail, "conv tail", torch.float32, 3)
+        if tuple(tail.shape[1:]) != (num_taps - 1, C):
+            raise KernelError("channel_delta_prepare: the tail does not fit the channels")
+    _need(rate_log, "rate_log", torch.float32, 1)
+    _need(rate_bias, "rate_bias", torch.float32, 1)
+    for t, what in ((tok_req, "tok_req"), (q_offsets, "q_offsets"), (slot_ids, "slot_ids")):
+        _need(t, what, torch.int32, 1)
+    if rate_log.shape[0] != heads or rate_bias.shape[0] != nk or tok_req.shape[0] != T:
+        raise KernelError("channel_delta_prepare: the decay's vectors or the token map do not fit")
+    coef = torch.empty((5, T, nk), dtype=torch.float32, device=proj.device)
+    v = torch.empty((T, heads * value_dim), dtype=torch.float32, device=proj.device)
+    if T:
+        _call("lc_channel_delta_prepare", _ptr(proj), proj.shape[1], int(beta_column), _ptr(rates), rates.shape[1],
+              int(rate_column), T, heads, kv_heads, key_dim, value_dim, num_taps, _ptr(taps),
+              _ptr(tail if num_taps > 1 else None), tail.shape[0] if num_taps > 1 else 0, _ptr(rate_log),
+              _ptr(rate_bias), float(unit_eps), _ptr(tok_req), _ptr(q_offsets), _ptr(slot_ids), _ptr(coef), _ptr(v),
+              _stream())
+    return coef, v
+
+
 def conv_tail_update(proj: torch.Tensor, tail: torch.Tensor, channels: int, num_taps: int,
                      q_offsets: torch.Tensor, slot_ids: torch.Tensor, num_requests: int) -> None:
     """After a step: ``tail`` [slots, K - 1, C] of every request of the batch becomes the last K - 1
@@ -1816,6 +1965,27 @@ def lightning_prepare(proj: torch.Tensor, heads: int, key_dim: int, value_dim: i
     return coef, v
 
 
+def gated_linear_prepare(proj: torch.Tensor, rates: torch.Tensor, rate_column: int, bias: torch.Tensor, power: float,
+                         q_scale: float, heads: int, key_dim: int, value_dim: int):
+    """The scan's inputs of gated linear attention from the float32 projections ``proj`` [T, >= heads (2 key_dim +
+    value_dim)]: columns q | k | v; z: the heads key_dim columns of float32 ``rates`` from ``rate_column`` on plus ``bias``.
+    Returns ``coef`` float32 [3, T, heads key_dim] (decay = sigmoid(z)^power per channel, write = k, read = ``q_scale``
+    q: no removal term) and ``v`` float32 [T, heads value_dim]."""
+    _need(proj, "gated_linear proj", torch.float32, 2)
+    _need(rates, "gated_linear rates", torch.float32, 2)
+    _need(bias, "gated_linear bias", torch.float32, 1)
+    T, nk = proj.shape[0], heads * key_dim
+    if proj.shape[1] < 2 * nk + heads * value_dim or rates.shape[0] != T or rate_column < 0 \
+            or rate_column + nk > rates.shape[1] or bias.shape[0] != nk:
+        raise KernelError("gated_linear_prepare: the projections or the bias do not fit the heads")
+    coef = torch.empty((3, T, nk), dtype=torch.float32, device=proj.device)
+    v = torch.empty((T, heads * value_dim), dtype=torch.float32, device=proj.device)
+    if T:
+        _call("lc_gated_linear_prepare", _ptr(proj), proj.shape[1], _ptr(rates), rates.shape[1], int(rate_column),
+              _ptr(bias), float(power), float(q_scale), T, heads, key_dim, value_dim, _ptr(coef), _ptr(v), _stream())
+    return coef, v
+
+
 def lightning_readout(o: torch.Tensor, gates: torch.Tensor, gate_column: int, weight: torch.Tensor, eps: float,
                       out_dtype: torch.dtype) -> torch.Tensor:
     """Every row of float32 ``o`` [T, n] (all heads side by side) divided by its root mean square (eps inside
@@ -1946,15 +2116,17 @@ def attention_prepare(proj: torch.Tensor, nq: int, nk: int, nv: int, d: int, dv:
 
 def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, tok_req: torch.Tensor,
                      positions: torch.Tensor, block_table: torch.Tensor, page_size: int, heads: int, kv_heads: int,
-                     maps: int, d: int, dv: int, scale: float, chunk: int = 0, window: int = 0,
-                     r1: Optional[torch.Tensor] = None, r2: Optional[torch.Tensor] = None,
+                     maps: int, d: int, dv: int, scale: float, chunk: int = 0, window: int = 0, keep: int = 0,
+                     cap: float = 0.0, r1: Optional[torch.Tensor] = None, r2: Optional[torch.Tensor] = None,
                      sink: Optional[torch.Tensor] = None, subtract: float = 0.0, unit_eps: Optional[float] = None,
                      out_scale: float = 1.0, gate: Optional[torch.Tensor] = None, gate_column: int = 0,
                      plan=None, max_ctx: int = 0) -> torch.Tensor:
     """Attention of every token of the batch over its request's cached keys lo .. p (p its position; lo the start
-    of its chunk of ``chunk`` positions, of its window of ``window``, or 0), float32 arithmetic.  ``q`` [T, heads
+    of its chunk of ``chunk`` positions, of its window of ``window``, or 0) and over the first ``keep`` of its keys
+    wherever lo is, float32 arithmetic.  ``q`` [T, heads
     maps d]; ``k_cache`` [pages, page, kv_heads maps d], ``v_cache`` [pages, page, kv_heads dv].  Scores are
-    ``scale`` (q . k) minus ``r1[h] ln(1 + r2[h] (p - j))`` where the bias is given; ``sink`` float32 [heads] adds
+    ``scale`` (q . k) minus ``r1[h] ln(1 + r2[h] (p - j))`` where the bias is given, then, where ``cap`` is positive,
+    cap tanh(score / cap); ``sink`` float32 [heads] adds
     exp(sink[h]) to the softmax's denominator.  ``maps`` = 2: a head's two maps over the same values are combined as
     a_0 - ``subtract`` a_1.  ``unit_eps``: the head's output is divided by its root mean square and multiplied by
     ``out_scale``.  ``gate`` float32 [T, >= gate_column + heads dv]: the output times sigmoid of those columns.
@@ -1990,21 +2162,21 @@ def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         # workgroup a CU in all), a workgroup keeping two blocks a wave at least
         zsplits, shares = 1, None
         if not plan.info.get("any_portion", True) and max_ctx > 0:
-            reach = min(int(chunk) or max_ctx, int(window) or max_ctx, max_ctx)
+            reach = min(min(int(chunk) or max_ctx, int(window) or max_ctx) + int(keep), max_ctx)
             zsplits = max(1, min(_masked_splits.forced or 256 // max(1, tiles.shape[0] * kv_heads), 16, reach // 256))
             if zsplits > 1:
                 words = library().lc_masked_attention_bf16_workspace(tiles.shape[0], heads, kv_heads, maps, dv, zsplits)
                 shares = torch.empty((words,), dtype=torch.float32, device=q.device)
         _call("lc_masked_attention_bf16", _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(tiles), tiles.shape[0],
               _ptr(block_table), block_table.shape[1], int(page_size), heads, kv_heads, maps, d, dv, float(scale),
-              int(chunk), int(window), _ptr(r1), _ptr(r2), _ptr(sink), float(subtract), 0 if unit_eps is None else 1,
+              int(chunk), int(window), int(keep), float(cap), _ptr(r1), _ptr(r2), _ptr(sink), float(subtract), 0 if unit_eps is None else 1,
               float(unit_eps or 0.0), float(out_scale), _ptr(gate), gate.shape[1] if gate is not None else 0,
               int(gate_column), _ptr(out), _ptr(shares), zsplits, 1 if plan.info.get("any_portion", True) else 0,
               1 if plan.info.get("any_lone", True) else 0, _stream())
     elif T:
         _call("lc_masked_attention", _ptr(q), _ptr(k_cache), _ptr(v_cache), _dt(q), _ptr(tok_req), _ptr(positions),
               _ptr(block_table), block_table.shape[1], int(page_size), T, heads, kv_heads, maps, d, dv, float(scale),
-              int(chunk), int(window), _ptr(r1), _ptr(r2), _ptr(sink), float(subtract), 0 if unit_eps is None else 1,
+              int(chunk), int(window), int(keep), float(cap), _ptr(r1), _ptr(r2), _ptr(sink), float(subtract), 0 if unit_eps is None else 1,
               float(unit_eps or 0.0), float(out_scale), _ptr(gate), gate.shape[1] if gate is not None else 0,
               int(gate_column), _ptr(out), _stream())
     return out
@@ -2149,6 +2321,62 @@ def attention_rows(proj: torch.Tensor, nq: int, nk: int, nv: int, d: int, dv: in
               float(eps), _ptr(table), rot, 1 if half else 0, _ptr(positions), _ptr(mix_from), float(mix), _ptr(values),
               _ptr(q), _ptr(k_cache), _ptr(v_cache), _dt(q), _ptr(rows), page, _stream())
     return q, values
+
+
+# ------------------------------------------------------------------------------ attention, every head on its own
+def attention_heads(proj: torch.Tensor, nq: int, nk: int, nv: int, d: int, dv: int, out_dtype: torch.dtype,
+                    k_cache: torch.Tensor, v_cache: torch.Tensor, rows: Optional[torch.Tensor],
+                    values_are_keys: bool = False, bias: Optional[torch.Tensor] = None,
+                    q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None, eps: float = 0.0,
+                    table: Optional[torch.Tensor] = None, rot: int = 0, half: bool = True,
+                    positions: Optional[torch.Tensor] = None,
+                    temperature: Optional[Tuple[float, float]] = None) -> torch.Tensor:
+    """q for the attention kernels, and k and v into their cache rows, from the float32 projections ``proj`` [T,
+    cols]: columns q (nq heads of d) | k (nk of d) | v (nv of dv), or q | k alone with ``values_are_keys`` (the values
+    are then k with its bias, before anything else).  ``bias`` float32 over these columns is added first; ``q_weight``
+    and ``k_weight`` [d]: every q (k) head divided by its root mean square (``eps`` inside the root) and weighed, one
+    weight for all heads; ``table`` [positions, rot]: the first ``rot`` entries of every q and k head are rotated,
+    entry i with i + rot/2 (``half``) or 2i with 2i + 1; ``temperature`` (coef, every): q at position p times 1 +
+    coef ln(floor((p + 1) / every) + 1).  ``rows``, ``k_cache`` and ``v_cache`` as for :func:`attention_rows`.
+    -> q [T, nq d] of ``out_dtype``."""
+    _need(proj, "attention_heads proj", torch.float32, 2)
+    T, cols = proj.shape
+    C = (nq + nk) * d + (0 if values_are_keys else nv * dv)
+    if cols < C:
+        raise KernelError(f"attention_heads: {cols} columns, the heads need {C}")
+    if values_are_keys and (nv, dv) != (nk, d):
+        raise KernelError("attention_heads: values that are the keys have the keys' heads and sizes")
+    if max(d, dv) > MASKED_ATTENTION_MAX:
+        raise KernelError(f"attention_heads: heads of {d}/{dv} entries are above {MASKED_ATTENTION_MAX}")
+    _need(k_cache, "key cache", out_dtype, 3)
+    _need(v_cache, "value cache", out_dtype, 3)
+    page = k_cache.shape[1]
+    if k_cache.shape[2] != nk * d or v_cache.shape[1] != nv * dv or v_cache.shape[2] != page:
+        raise KernelError("attention_heads: the caches do not fit the heads")
+    for t, what, n in ((bias, "bias", C), (q_weight, "q weight", d), (k_weight, "k weight", d)):
+        if t is not None:
+            _need(t, f"attention_heads {what}", torch.float32, 1)
+            if t.shape[0] != n:
+                raise KernelError(f"attention_heads: the {what} has {t.shape[0]} entries, expected {n}")
+    if rows is not None:
+        _need(rows, "attention_heads rows", torch.int32, 1)
+        if rows.shape[0] != T:
+            raise KernelError("attention_heads: one place per token")
+    if table is not None:
+        _need(table, "rotary table", torch.float32, 2)
+        if table.shape[1] != rot or rot % 2 or rot > d:
+            raise KernelError("attention_heads: the rotary table does not fit")
+    coef, every = temperature if temperature is not None else (0.0, 0.0)
+    if table is not None or temperature is not None:
+        _need(positions, "positions", torch.int32, 1)
+        if positions.shape[0] != T:
+            raise KernelError("attention_heads: one position per token")
+    q = torch.empty((T, nq * d), dtype=out_dtype, device=proj.device)
+    if T:
+        _call("lc_attention_heads", _ptr(proj), cols, T, nq, nk, nv, d, dv, 1 if values_are_keys else 0, _ptr(bias),
+              _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(table), int(rot), 1 if half else 0, _ptr(positions),
+              float(coef), float(every), _ptr(q), _ptr(k_cache), _ptr(v_cache), _dt(q), _ptr(rows), page, _stream())
+    return q
 
 
 # ------------------------------------------------------------------------------ matrix memory (mLSTM)

@@ -48,6 +48,47 @@ class PreNormMixerBlock:
         stream.pending = self.mixer.forward(x, site)
 
 
+@BLOCKS.register("parallel_residual")
+class ParallelResidualBlock:
+    """Both branches read the same stream, each behind a norm of its own: h = h + mixer(norm_1(h)) +
+    feed_forward(norm_2(h)).  The two norms divide by one root mean square: a norm that can (``add_norm_pair``) makes
+    both rows in the kernel that adds what waits.  The branches wait together (``ops.SummedBranches``); a branch that is
+    itself several hands them over unadded (``forward_branches``)."""
+
+    slots = {"mixer": "mixer", "feed_forward": "feed_forward", "mixer_norm": "norm", "feed_forward_norm": "norm"}
+
+    def __init__(self, mixer, feed_forward, mixer_norm, feed_forward_norm):
+        self.mixer, self.feed_forward = mixer, feed_forward
+        self.mixer_norm, self.feed_forward_norm = mixer_norm, feed_forward_norm
+        self.paired = hasattr(mixer_norm, "add_norm_pair") and mixer_norm.pairs_with(feed_forward_norm)
+
+    def forward(self, stream: ResidualStream, site) -> None:
+        from ..kernels import ops
+        if self.paired:
+            x, z = self.mixer_norm.add_norm_pair(stream, self.feed_forward_norm)
+        else:
+            x = self.mixer_norm.add_norm(stream)
+            z = self.feed_forward_norm.add_norm(stream)         # nothing waits any more: the same stream
+        y = getattr(self.mixer, "forward_branches", self.mixer.forward)(x, site)
+        f = getattr(self.feed_forward, "forward_branches", self.feed_forward.forward)(z)
+        stream.pending = ops.summed((y, 1.0), (f, 1.0))
+
+
+@BLOCKS.register("parallel_mixer")
+class ParallelMixerBlock:
+    """The same without a feed-forward: h = h + mixer(norm(h)), a mixer's several branches handed over unadded."""
+
+    slots = {"mixer": "mixer", "mixer_norm": "norm"}
+
+    def __init__(self, mixer, mixer_norm):
+        self.mixer, self.mixer_norm = mixer, mixer_norm
+
+    def forward(self, stream: ResidualStream, site) -> None:
+        from ..kernels import ops
+        x = self.mixer_norm.add_norm(stream)
+        stream.pending = ops.summed((getattr(self.mixer, "forward_branches", self.mixer.forward)(x, site), 1.0))
+
+
 def _caching_index(parts, part) -> int:
     """Which of the site's caches belongs to ``part``: a site's caches follow the layer's caching parts
     in the order of the block's slots."""

@@ -19,6 +19,10 @@ SiLU; q and k are made unit vectors, q times key_dim^(-1/2); one decay g = exp(-
 + k u^T is the recurrence above with decay = g, probe = g k, removal = beta k, write = beta k.  The
 last ``taps - 1`` inputs of the convolutions are state as well.
 
+``channel_delta`` (the gated delta rule with a decay per key channel): the same with g = exp(-exp(A_head) softplus(W_a2
+(W_a1 h) + b)) per head and key channel, and an output gate sigmoid(W_g2 (W_g1 h)).  S <- diag(g) S; u = beta (v - S^T k);
+S <- S + k u^T is the recurrence above with decay = g, probe = g k (channel by channel), removal = beta k, write = beta k.
+
 Everything between the projections and the output product is float32: the projections leave as
 float32, a kernel turns them into the five vectors (gates, exponentials, unit vectors), the scan
 keeps S in float32, and the read-out is divided by its root mean square per head and gated before
@@ -36,7 +40,7 @@ from ..config.registry import MIXERS
 from ..kernels import ops
 from ..weights.loader import ParamDecl
 from .base import BuildContext, Part
-from .feed_forward import stack_rows
+from .feed_forward import low_rank, stack_rows
 
 
 def _f32(t: torch.Tensor) -> torch.Tensor:
@@ -142,4 +146,62 @@ class GatedDelta(Part):
                            self.nh, self.dk, self.dv)
         y = ops.head_gate_norm(o, proj, self.channels, self.norm, False, self.norm_eps, "silu", self.nh, self.dv,
                                self.dtype)
+        return ops.gemm(y, self.o, self.dtype, defer=True)
+
+
+@MIXERS.register("channel_delta")
+class ChannelDelta(Part):
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, key_dim: int, value_dim: int,
+                 conv_taps: int, norm_eps: float, unit_eps: float = 1e-6):
+        super().__init__(hidden_size=hidden_size, num_heads=num_heads, num_kv_heads=num_kv_heads, key_dim=key_dim,
+                         value_dim=value_dim, conv_taps=conv_taps, norm_eps=norm_eps, unit_eps=unit_eps)
+        if num_heads % num_kv_heads:
+            raise ValueError(f"channel_delta: {num_heads} heads are not a multiple of {num_kv_heads} kv heads")
+        self.H, self.nh, self.nkv = int(hidden_size), int(num_heads), int(num_kv_heads)
+        self.dk, self.dv, self.taps = int(key_dim), int(value_dim), int(conv_taps)
+        self.norm_eps, self.unit_eps = float(norm_eps), float(unit_eps)
+        self.channels = 2 * self.nkv * self.dk + self.nh * self.dv       # what passes the convolutions
+        ops.check_delta_sizes("channel_delta", self.dk, self.dv, self.taps)
+
+    def declare(self) -> Dict[str, ParamDecl]:
+        nq, nk, nv = self.nkv * self.dk, self.nh * self.dk, self.nh * self.dv
+        # the inner sizes of the decay's and the gate's two matrices are whatever the checkpoint holds
+        return {"q": ParamDecl((nq, self.H)), "q_conv": ParamDecl((nq, self.taps), role="vector"),
+                "k": ParamDecl((nq, self.H)), "k_conv": ParamDecl((nq, self.taps), role="vector"),
+                "v": ParamDecl((nv, self.H)), "v_conv": ParamDecl((nv, self.taps), role="vector"),
+                "beta": ParamDecl((self.nh, self.H)), "rate_log": ParamDecl((self.nh,), role="vector"),
+                "rate_in": ParamDecl((-1, self.H)), "rate_out": ParamDecl((nk, -1)),
+                "rate_bias": ParamDecl((nk,), role="vector"),
+                "gate_in": ParamDecl((-1, self.H)), "gate_out": ParamDecl((nv, -1)),
+                "norm": ParamDecl((self.dv,), role="vector", init="ones_plus_normal"), "o": ParamDecl((self.H, nv))}
+
+    def bind(self, tensors, ctx: BuildContext) -> None:
+        self.dtype = ctx.dtype
+        self.proj = stack_rows([tensors[k] for k in ("q", "k", "v", "beta")])
+        self.inner, self.outer = low_rank((tensors["rate_in"], tensors["gate_in"]),
+                                          (tensors["rate_out"], tensors["gate_out"]), ctx.dtype == torch.bfloat16)
+        self.conv = torch.cat([_f32(tensors[k]) for k in ("q_conv", "k_conv", "v_conv")], dim=0).contiguous()
+        self.rate_log, self.rate_bias = _f32(tensors["rate_log"]), _f32(tensors["rate_bias"])
+        self.norm, self.o = _f32(tensors["norm"]), tensors["o"]
+
+    def cache_need(self):
+        return FixedStates(((self.nh, self.dv, self.dk), (max(self.taps - 1, 0), self.channels)))
+
+    def forward(self, x: torch.Tensor, site) -> torch.Tensor:
+        batch = site.batch
+        state, tail = site.cache
+        proj = ops.gemm(x, self.proj, torch.float32)
+        # columns: the decay's inputs, head by head and channel by channel, then the output gate's
+        gates = ops.gemm(ops.gemm(x, self.inner, self.dtype), self.outer, torch.float32)
+        coef, v = ops.channel_delta_prepare(proj, self.channels, gates, 0, tail, self.conv, self.rate_log,
+                                            self.rate_bias, self.nh, self.nkv, self.dk, self.dv, self.taps,
+                                            self.unit_eps, batch.tok_req, batch.q_offsets, batch.slot_ids)
+        ops.conv_tail_update(proj, tail, self.channels, self.taps, batch.q_offsets, batch.slot_ids,
+                             batch.num_requests)
+        o = ops.delta_scan(coef, v, state, batch.q_offsets, batch.slot_ids, batch.num_requests,
+                           self.nh, self.dk, self.dv)
+        y = ops.head_gate_norm(o, gates, self.nh * self.dk, self.norm, False, self.norm_eps, "sigmoid", self.nh,
+                               self.dv, self.dtype)
         return ops.gemm(y, self.o, self.dtype, defer=True)

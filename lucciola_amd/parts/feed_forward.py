@@ -20,6 +20,29 @@ def _softplus(z: float) -> float:
     return math.log1p(math.exp(-abs(z))) + max(z, 0.0)
 
 
+INNER_MULTIPLE = 128        # what the matrix-core products want of a product's inner size
+
+
+def low_rank(inner, outer, pad: bool):
+    """Several pairs of small matrices, outer_k (inner_k x), as two products: the inner matrices stacked, and the outer
+    ones on the diagonal of one matrix (zeros elsewhere).  ``pad``: zero rows bring the inner size to a multiple of
+    INNER_MULTIPLE.  -> (inner [r, n], outer [sum of outer rows, r])"""
+    for a, b in zip(inner, outer):
+        if b.shape[1] != a.shape[0]:
+            raise ValueError(f"the two matrices of a low-rank product do not fit each other ({tuple(a.shape)}, {tuple(b.shape)})")
+    rank = sum(a.shape[0] for a in inner)
+    size = -(-rank // INNER_MULTIPLE) * INNER_MULTIPLE if pad else rank
+    first = stack_rows(list(inner))
+    second = first.new_zeros((sum(b.shape[0] for b in outer), size))
+    row = column = 0
+    for b in outer:
+        second[row:row + b.shape[0], column:column + b.shape[1]] = b.to(second.dtype)
+        row, column = row + b.shape[0], column + b.shape[1]
+    if size > rank:
+        first = torch.cat([first, first.new_zeros((size - rank, first.shape[1]))]).contiguous()
+    return first, second
+
+
 def stack_rows(tensors):
     """Stack weight matrices along their rows; mixed storage widens to float32."""
     dtypes = {t.dtype for t in tensors}
@@ -82,7 +105,7 @@ class GatedMLP(Part):
 @FEED_FORWARDS.register("mlp")
 class MLP(Part):
     """The plain two-matrix feed-forward ``down(act(up(x)))``, no biases.  ``activation``:
-    "gelu_tanh" (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))), "relu_squared", or "xielu": with two
+    "gelu_tanh" (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))), "gelu" (0.5 z (1 + erf(z / sqrt(2)))), "relu_squared", or "xielu": with two
     learned numbers p, q (tensor ``act``), z > 0: softplus(p) z^2 + z/2; z <= 0: (1/2 + softplus(q))
     (e^z - 1 - z) + z/2."""
 
@@ -138,7 +161,7 @@ class RoutedMLP(Part):
                          top=top, activation=activation, scores=scores, renormalise=renormalise,
                          renormalise_eps=renormalise_eps, correction=correction, groups=groups,
                          keep_groups=keep_groups, weight_scale=weight_scale)
-        if activation not in ("gelu_tanh", "relu_squared"):
+        if activation not in ("gelu_tanh", "gelu", "relu_squared"):
             raise ValueError(f"routed_mlp: activation '{activation}' has no kernel")
         if scores not in ("softmax", "sigmoid"):
             raise ValueError(f"routed_mlp: scores '{scores}' have no kernel (softmax, sigmoid)")
@@ -176,6 +199,11 @@ class RoutedMLP(Part):
         self.large_tiles = ctx.device.type == "cuda" and ops.moe_large_tiles(ctx.dtype, self.up, self.down)
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return self.forward_branches(x).value()
+
+    def forward_branches(self, x: torch.Tensor) -> ops.RoutedRows:
+        """The experts' rows before they are weighed and added, for a block that does so in the kernel that adds them
+        to its stream."""
         logits = ops.gemm(x, self.router, torch.float32)
         if self.scores == "sigmoid":
             routing = ops.moe_route_sigmoid(logits, self.top, self.correction_vector, self.groups, self.keep_groups,
@@ -184,8 +212,7 @@ class RoutedMLP(Part):
             routing = ops.moe_route(logits, self.top, self.renormalise, self.renormalise_eps,
                                     large_tiles=self.large_tiles)
         hidden = ops.moe_experts(x, self.up, routing, self.dtype, activation=self.activation, gather=True)
-        y = ops.moe_experts(hidden, self.down, routing, torch.float32)
-        return ops.moe_combine(y, routing, self.dtype)
+        return ops.RoutedRows(ops.moe_experts(hidden, self.down, routing, torch.float32), routing, self.dtype)
 
 
 @FEED_FORWARDS.register("routed_gated_mlp")

@@ -15,24 +15,34 @@
   token, (1 - lambda) v + lambda v_earlier with one learned number (tensor ``vmix``), before they are cached:
   "keep": the values as projected stay for later layers of the pass; "mix": they are mixed with those that the last
   "keep" layer before this one left (a "keep" layer has the tensor too and does not use it);
+  or "keys": there is no value projection, the values are the keys as projected (bias included, before any norm or
+  rotation);
+- ``output_bias`` False: biases on q, k and v only;
+- ``head_norm``: every q head is divided by its root mean square and multiplied by a weight of the head's size that all
+  heads share, and so is every k head with another one, before the rotation;
+- ``temperature`` (coef, every): q at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1);
 - ``unit_qk``: every q and k head is divided by its root mean square (no weight);
 - ``distance_bias``: r1_h ln(1 + r2_h (i - j)) is taken off the score of query i and key j (two learned numbers a
   head);
-- ``sink``: a learned number s_h a head whose exp(s_h) is one more term of the softmax's denominator;
+- ``softcap``: the scores become softcap tanh(score / softcap);
+- ``sink``: a learned number s_h a head whose exp(s_h) is one more term of the softmax's denominator; or a number, the
+  same constant for every head (0.0: one is added to the denominator) and no tensor;
 - ``gate``: the heads' outputs times sigmoid(W_g h), entry by entry, before the output projection;
 - ``chunk``: position i sees j <= i only inside its own chunk of that many positions, counted from the sequence's
-  start; ``window``: only the last so many positions.
+  start; ``window``: only the last so many positions; ``keep_first``: the first so many positions are seen
+  by every later one beside those (their pages are not given back).
 
 The projections leave as float32; one kernel makes q, k and v of them (convolution, rotation of interleaved pairs,
 unit norm; or, with ``bias``, ``row_norm``, ``values`` or rotation of halves, the kernel that knows those:
-``ops.attention_rows``) and writes k and v into the cache (keys token-major, values transposed inside a page).  Scores, softmax, bias, sink
+``ops.attention_rows``; or, with ``head_norm``, ``temperature`` or values that are the keys, ``ops.attention_heads``) and
+writes k and v into the cache (keys token-major, values transposed inside a page).  Scores, softmax, bias, sink
 and the maps' combination are float32 whatever the cache's type; with a bfloat16 cache of sizes that fit, the two
 products run on the matrix cores (``ops.masked_attention``), else in float32 multiply-adds.
 """
 from __future__ import annotations
 
 import math
-from typing import Dict, Optional
+from typing import Dict, Optional, Sequence, Union
 
 import torch
 
@@ -59,13 +69,16 @@ class MaskedAttention(Part):
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
                  scale: float, eps: float, maps: int = 1, difference: float = 0.0, conv_taps: int = 0,
                  position: Optional[PartSpec] = None, unit_qk: bool = False, distance_bias: bool = False,
-                 sink: bool = False, gate: bool = False, chunk: Optional[int] = None, window: Optional[int] = None,
-                 bias: bool = False, row_norm: bool = False, values: Optional[str] = None):
+                 sink: Union[bool, float] = False, gate: bool = False, chunk: Optional[int] = None,
+                 window: Optional[int] = None, bias: bool = False, row_norm: bool = False, values: Optional[str] = None,
+                 output_bias: bool = True, head_norm: bool = False, temperature: Optional[Sequence[float]] = None,
+                 softcap: float = 0.0, keep_first: int = 0):
         super().__init__(hidden_size=hidden_size, num_heads=num_heads, num_kv_heads=num_kv_heads, head_dim=head_dim,
                          value_dim=value_dim, scale=scale, eps=eps, maps=maps, difference=difference,
                          conv_taps=conv_taps, position=position, unit_qk=unit_qk, distance_bias=distance_bias,
                          sink=sink, gate=gate, chunk=chunk, window=window, bias=bias, row_norm=row_norm,
-                         values=values)
+                         values=values, output_bias=output_bias, head_norm=head_norm, temperature=temperature,
+                         softcap=softcap, keep_first=keep_first)
         if num_heads % num_kv_heads:
             raise ValueError(f"masked_attention: {num_heads} heads are not a multiple of {num_kv_heads} kv heads")
         if maps not in (1, 2):
@@ -79,19 +92,35 @@ class MaskedAttention(Part):
         self.taps = int(conv_taps)
         if not 0 <= self.taps <= ops.SHORT_CONV_MAX_TAPS:
             raise ValueError(f"masked_attention: {self.taps} taps are above the kernel's {ops.SHORT_CONV_MAX_TAPS}")
+        # a sink of one constant for all heads is no tensor
+        self.sink_constant = None if isinstance(sink, bool) else float(sink)
         self.unit_qk, self.distance_bias, self.has_sink, self.has_gate = (bool(unit_qk), bool(distance_bias),
-                                                                          bool(sink), bool(gate))
+                                                                          sink is True, bool(gate))
         self.chunk, self.window = int(chunk) if chunk else 0, int(window) if window else 0
+        self.keep_first, self.softcap = int(keep_first), float(softcap)
+        if self.keep_first < 0 or self.softcap < 0:
+            raise ValueError("masked_attention: keep_first and softcap must not be negative")
         self.position = build_part(POSITION_ENCODINGS, position) if position else None
         self.has_bias, self.row_norm, self.values = bool(bias), bool(row_norm), values
-        if values not in (None, "keep", "mix"):
-            raise ValueError(f"masked_attention: values '{values}' are neither 'keep' nor 'mix'")
+        if values not in (None, "keep", "mix", "keys"):
+            raise ValueError(f"masked_attention: values '{values}' are neither 'keep' nor 'mix' nor 'keys'")
+        self.has_output_bias, self.head_norm = self.has_bias and bool(output_bias), bool(head_norm)
+        self.temperature = tuple(float(v) for v in temperature) if temperature is not None else None
+        if self.temperature is not None and (len(self.temperature) != 2 or not self.temperature[1] > 0):
+            raise ValueError("masked_attention: a temperature is (coef, every) with every > 0")
+        self.values_are_keys = values == "keys"
+        if self.values_are_keys and self.dv != self.d:
+            raise ValueError(f"masked_attention: values that are the keys have {self.d} entries, not {self.dv}")
         pairing = getattr(self.position, "pairing", None)
         if self.position is not None and pairing not in ("half", "interleaved"):
             raise ValueError(f"masked_attention: no prologue kernel rotates with the pairing '{pairing}'")
         self.half = pairing == "half"
-        # which of the two prologue kernels makes q, k and v
-        self.by_rows = self.has_bias or self.row_norm or self.values is not None or self.half
+        # which of the prologue kernels makes q, k and v
+        self.by_heads = self.head_norm or self.temperature is not None or self.values_are_keys
+        self.by_rows = not self.by_heads and (self.has_bias or self.row_norm or self.values is not None or self.half)
+        if self.by_heads and (self.row_norm or self.taps or self.unit_qk or self.maps > 1 or values in ("keep", "mix")):
+            raise ValueError("masked_attention: head_norm, temperature and values that are the keys go without row_norm, "
+                             "convolutions, unit_qk, several maps and mixed values (no prologue kernel has both)")
         if self.by_rows and (self.taps or self.unit_qk):
             raise ValueError("masked_attention: convolutions and unit_qk go without bias, row_norm, values and "
                              "rotation of halves (no prologue kernel has both)")
@@ -101,11 +130,14 @@ class MaskedAttention(Part):
         self.nq_cols = self.nh * self.maps * self.d
         self.nk_cols = self.nkv * self.maps * self.d
         self.nv_cols = self.nkv * self.dv
-        self.channels = self.nq_cols + self.nk_cols + self.nv_cols      # what passes the convolutions
+        # columns of the projection: q | k | v, or q | k where the values are the keys (what passes the convolutions)
+        self.channels = self.nq_cols + self.nk_cols + (0 if self.values_are_keys else self.nv_cols)
 
     def declare(self) -> Dict[str, ParamDecl]:
         out = {"q": ParamDecl((self.nq_cols, self.H)), "k": ParamDecl((self.nk_cols, self.H)),
                "v": ParamDecl((self.nv_cols, self.H)), "o": ParamDecl((self.H, self.nh * self.dv))}
+        if self.values_are_keys:
+            del out["v"]
         if self.taps:
             out.update({"q_conv": ParamDecl((self.nq_cols, self.taps), role="vector"),
                         "k_conv": ParamDecl((self.nk_cols, self.taps), role="vector"),
@@ -123,17 +155,22 @@ class MaskedAttention(Part):
         if self.has_bias:
             for name, size in (("q_bias", self.nq_cols), ("k_bias", self.nk_cols), ("v_bias", self.nv_cols),
                                ("o_bias", self.H)):
-                out[name] = ParamDecl((size,), role="vector")
+                if (name != "v_bias" or not self.values_are_keys) and (name != "o_bias" or self.has_output_bias):
+                    out[name] = ParamDecl((size,), role="vector")
         if self.row_norm:
             out["q_norm"] = ParamDecl((self.nq_cols,), role="vector", init="ones_plus_normal")
             out["k_norm"] = ParamDecl((self.nk_cols,), role="vector", init="ones_plus_normal")
-        if self.values is not None:
+        if self.head_norm:
+            out["q_norm"] = ParamDecl((self.d,), role="vector", init="ones_plus_normal")
+            out["k_norm"] = ParamDecl((self.d,), role="vector", init="ones_plus_normal")
+        if self.values in ("keep", "mix"):
             out["vmix"] = ParamDecl((), role="vector")
         return out
 
     def bind(self, tensors, ctx: BuildContext) -> None:
         self.dtype = ctx.dtype
-        mats = [tensors["q"], tensors["k"], tensors["v"]] + ([tensors["g"]] if self.has_gate else [])
+        projected = ("q", "k") if self.values_are_keys else ("q", "k", "v")
+        mats = [tensors[k] for k in projected] + ([tensors["g"]] if self.has_gate else [])
         self.proj = stack_rows(mats)
         self.o = tensors["o"]
         self.conv = None
@@ -147,11 +184,13 @@ class MaskedAttention(Part):
         self.r1 = _f32(tensors["r1"]) if self.distance_bias else None
         self.r2 = _f32(tensors["r2"]) if self.distance_bias else None
         self.sink = _f32(tensors["sink"]) if self.has_sink else None
+        if self.sink_constant is not None:
+            self.sink = torch.full((self.nh,), self.sink_constant, dtype=torch.float32, device=ctx.device)
         self.bias = self.o_bias = self.q_norm = self.k_norm = None
         if self.has_bias:
-            self.bias = torch.cat([_f32(tensors[k]) for k in ("q_bias", "k_bias", "v_bias")]).contiguous()
-            self.o_bias = _f32(tensors["o_bias"])
-        if self.row_norm:
+            self.bias = torch.cat([_f32(tensors[k + "_bias"]) for k in projected]).contiguous()
+            self.o_bias = _f32(tensors["o_bias"]) if self.has_output_bias else None
+        if self.row_norm or self.head_norm:
             self.q_norm, self.k_norm = _f32(tensors["q_norm"]), _f32(tensors["k_norm"])
         # one number for the layer; read once, at load
         self.mix = float(tensors["vmix"].to(torch.float32).item()) if self.values == "mix" else 0.0
@@ -159,7 +198,8 @@ class MaskedAttention(Part):
             self.position.bind({}, ctx)
 
     def cache_need(self):
-        rows = PagedRows(self.nk_cols, self.nv_cols, self.window or None)
+        rows = PagedRows(self.nk_cols, self.nv_cols, self.window or None,
+                         self.keep_first if self.window else 0)
         if self.taps > 1:
             return rows, FixedStates(((self.taps - 1, self.channels),))
         return rows
@@ -184,23 +224,34 @@ class MaskedAttention(Part):
         table, rot = None, 0
         if self.position is not None:
             table, rot = self.position.rotary_table(batch.max_position), self.position.rotary_dim
-        q = self._by_rows(proj, site, k_cache, v_cache, table, rot) if self.by_rows else ops.attention_prepare(
-            proj, self.nh * self.maps, self.nkv * self.maps, self.nkv, self.d, self.dv, self.dtype,
-            k_cache, v_cache, pages.slots if site.writes_cache else None,
-            taps=self.conv, tail=tail, tok_req=batch.tok_req, q_offsets=batch.q_offsets, slot_ids=batch.slot_ids,
-            table=table, rot=rot, positions=batch.positions, unit_eps=self.eps if self.unit_qk else None)
+        slots = pages.slots if site.writes_cache else None
+        if self.by_heads:
+            q = ops.attention_heads(
+                proj, self.nh, self.nkv, self.nkv, self.d, self.dv, self.dtype, k_cache, v_cache, slots,
+                values_are_keys=self.values_are_keys, bias=self.bias, q_weight=self.q_norm, k_weight=self.k_norm,
+                eps=self.eps, table=table, rot=rot, half=self.half, positions=batch.positions,
+                temperature=self.temperature)
+        elif self.by_rows:
+            q = self._by_rows(proj, site, k_cache, v_cache, table, rot)
+        else:
+            q = ops.attention_prepare(
+                proj, self.nh * self.maps, self.nkv * self.maps, self.nkv, self.d, self.dv, self.dtype, k_cache, v_cache,
+                slots, taps=self.conv, tail=tail, tok_req=batch.tok_req, q_offsets=batch.q_offsets,
+                slot_ids=batch.slot_ids, table=table, rot=rot, positions=batch.positions,
+                unit_eps=self.eps if self.unit_qk else None)
         if self.taps > 1:
             ops.conv_tail_update(proj, tail, self.channels, self.taps, batch.q_offsets, batch.slot_ids,
                                  batch.num_requests)
         o = ops.masked_attention(
             q, k_cache, v_cache, batch.tok_req, batch.positions, pages.block_table, pages.page_size, self.nh, self.nkv,
-            self.maps, self.d, self.dv, self.scale, chunk=self.chunk, window=self.window, r1=self.r1, r2=self.r2,
+            self.maps, self.d, self.dv, self.scale, chunk=self.chunk, window=self.window,
+            keep=self.keep_first if self.window or self.chunk else 0, cap=self.softcap, r1=self.r1, r2=self.r2,
             sink=self.sink, subtract=self.subtract, unit_eps=self.eps if self.maps == 2 else None,
             out_scale=1.0 - self.difference if self.maps == 2 else 1.0,
             gate=proj if self.has_gate else None, gate_column=self.channels, plan=batch.plans.get(ops.LATENT_PLAN),
             max_ctx=batch.max_ctx)
         y = ops.gemm(o, self.o, self.dtype, defer=True)
-        return ops.BiasedBranch(y, self.o_bias) if self.has_bias else y
+        return ops.BiasedBranch(y, self.o_bias) if self.o_bias is not None else y
 
     def _by_rows(self, proj: torch.Tensor, site, k_cache, v_cache, table, rot: int) -> torch.Tensor:
         batch, earlier = site.batch, None

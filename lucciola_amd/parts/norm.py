@@ -50,6 +50,16 @@ class RMSNorm(Part):
         stream.pending = None
         return x
 
+    def pairs_with(self, other) -> bool:
+        """Whether one pass can norm the stream for this norm and ``other``: the same root mean square."""
+        return isinstance(other, RMSNorm) and (other.size, other.eps) == (self.size, self.eps)
+
+    def add_norm_pair(self, stream: ResidualStream, other: "RMSNorm") -> Tuple[torch.Tensor, torch.Tensor]:
+        """Add what waits into the stream; the normed stream with this norm's weight and with ``other``'s."""
+        x, y = ops.stream_norms(stream.h, stream.pending, (self.weight, other.weight), self.eps, self.dtype)
+        stream.pending = None
+        return x, y
+
     def add_norm_rows(self, stream: ResidualStream, rows: torch.Tensor) -> torch.Tensor:
         """The normed stream (pending included) at the given rows only; the stream is not changed."""
         return ops.rmsnorm(stream.h, stream.pending, self.weight, self.eps, self.dtype, rows=rows)

@@ -60,9 +60,17 @@ class ParallelMixers(Part):
     def ready(self, position: int) -> bool:
         return self.left.ready(position) and self.right.ready(position)
 
-    def forward(self, x: torch.Tensor, site) -> torch.Tensor:
+    def _both(self, x: torch.Tensor, site):
         if isinstance(x, ops.ScaledRows):
             x = x.value()
-        a = self.left.forward(x, site.span(0, self._left_needs))
-        b = self.right.forward(x, site.span(self._left_needs, self._right_needs))
+        return (self.left.forward(x, site.span(0, self._left_needs)),
+                self.right.forward(x, site.span(self._left_needs, self._right_needs)))
+
+    def forward(self, x: torch.Tensor, site) -> torch.Tensor:
+        a, b = self._both(x, site)
         return ops.scaled_sum(a, self.left_scale, b, self.right_scale)
+
+    def forward_branches(self, x: torch.Tensor, site) -> ops.SummedBranches:
+        """The same for a block that adds several branches to its stream in one kernel."""
+        a, b = self._both(x, site)
+        return ops.summed((a, self.left_scale), (b, self.right_scale))

@@ -17,6 +17,8 @@ def embedding(ids, table, scale=1.0):
 
 
 def rmsnorm(h, delta, weight, eps, out_dtype, rows=None, scaled=False):   # never hands out scaled rows
+    if hasattr(delta, "branches"):          # several branches at once
+        return stream_norms(h, delta, (weight,), eps, out_dtype, rows=rows)[0]
     if hasattr(delta, "branch"):            # a branch and its bias
         delta = delta.branch.to(F64) + delta.bias.to(F64)
     if rows is None:
@@ -29,6 +31,18 @@ def rmsnorm(h, delta, weight, eps, out_dtype, rows=None, scaled=False):   # neve
             v = (h[rows.long()] + delta[rows.long()].to(torch.float32)).to(F64)
     inv = torch.rsqrt((v * v).mean(dim=-1, keepdim=True) + eps)
     return (v * inv * weight.to(F64)).to(out_dtype)
+
+
+def stream_norms(h, delta, weights, eps, out_dtype, rows=None):
+    v = h.to(F64)
+    for output, scale in () if delta is None else delta.branches if hasattr(delta, "branches") else ((delta, 1.0),):
+        v = v + scale * (output if isinstance(output, torch.Tensor) else output.value()).to(F64)
+    if rows is None:
+        h.copy_(v.to(torch.float32))
+    else:
+        v = v[rows.long()]
+    v = v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps)
+    return tuple((v * w.to(F64)).to(out_dtype) for w in weights)
 
 
 def rmsnorm_act(x, weight, eps, column=None):
@@ -182,6 +196,8 @@ def _act(z, kind, params=(0.0, 0.0)):
         return torch.where(z > 0, params[0] * z * z + 0.5 * z, params[1] * (torch.expm1(neg) - neg) + 0.5 * z)
     if kind == "gelu_tanh":
         return 0.5 * z * (1 + torch.tanh(math.sqrt(2 / math.pi) * (z + 0.044715 * z ** 3)))
+    if kind == "gelu":
+        return 0.5 * z * (1 + torch.erf(z / math.sqrt(2.0)))
     if kind == "relu_squared":
         return torch.clamp(z, min=0) ** 2
     raise ValueError(kind)
@@ -317,6 +333,14 @@ def lightning_prepare(proj, heads, key_dim, value_dim, decay):
     coef[1] = silu(p[:, nk:2 * nk])
     coef[2] = silu(p[:, :nk])
     return coef.to(torch.float32), silu(p[:, 2 * nk:2 * nk + nv]).to(torch.float32)
+
+
+def gated_linear_prepare(proj, rates, rate_column, bias, power, q_scale, heads, key_dim, value_dim):
+    nk, nv = heads * key_dim, heads * value_dim
+    p = proj.to(F64)
+    keep = torch.sigmoid(rates[:, rate_column:rate_column + nk].to(F64) + bias.to(F64)) ** power
+    coef = torch.stack([keep, p[:, nk:2 * nk], q_scale * p[:, :nk]])
+    return coef.to(torch.float32), p[:, 2 * nk:2 * nk + nv].to(torch.float32).contiguous()
 
 
 def lightning_readout(o, gates, gate_column, weight, eps, out_dtype):
@@ -488,6 +512,22 @@ def gated_delta_prepare(proj, tail, taps, rate_log, rate_bias, heads, kv_heads, 
     return coef.to(torch.float32).contiguous(), v.to(torch.float32).contiguous()
 
 
+def channel_delta_prepare(proj, beta_column, rates, rate_column, tail, taps, rate_log, rate_bias, heads, kv_heads, key_dim,
+                          value_dim, num_taps, unit_eps, tok_req, q_offsets, slot_ids):
+    T, nq, nk = proj.shape[0], kv_heads * key_dim, heads * key_dim
+    y = _convolved(proj, 2 * nq + heads * value_dim, taps, tail, tok_req, q_offsets, slot_ids)
+    y = y * torch.sigmoid(y)
+    q, k, v = y[:, :nq].view(T, kv_heads, key_dim), y[:, nq:2 * nq].view(T, kv_heads, key_dim), y[:, 2 * nq:]
+    q = q / torch.sqrt((q * q).sum(-1, keepdim=True) + unit_eps) * key_dim ** -0.5
+    k = k / torch.sqrt((k * k).sum(-1, keepdim=True) + unit_eps)
+    q, k = (x.repeat_interleave(heads // kv_heads, dim=1) for x in (q, k))
+    beta = torch.sigmoid(proj[:, beta_column:beta_column + heads].to(F64))[:, :, None]
+    step = torch.nn.functional.softplus(rates[:, rate_column:rate_column + nk].to(F64) + rate_bias.to(F64))
+    g = torch.exp(-torch.exp(rate_log.to(F64))[None, :, None] * step.view(T, heads, key_dim))
+    coef = torch.stack([g, g * k, beta * k, beta * k, q]).reshape(5, T, nk)
+    return coef.to(torch.float32).contiguous(), v.to(torch.float32).contiguous()
+
+
 def conv_tail_update(proj, tail, channels, num_taps, q_offsets, slot_ids, num_requests):
     if num_taps <= 1:
         return
@@ -596,7 +636,7 @@ def attention_prepare(proj, nq, nk, nv, d, dv, out_dtype, k_cache, v_cache, rows
 
 
 def masked_attention(q, k_cache, v_cache, tok_req, positions, block_table, page_size, heads, kv_heads, maps, d, dv,
-                     scale, chunk=0, window=0, r1=None, r2=None, sink=None, subtract=0.0, unit_eps=None,
+                     scale, chunk=0, window=0, keep=0, cap=0.0, r1=None, r2=None, sink=None, subtract=0.0, unit_eps=None,
                      out_scale=1.0, gate=None, gate_column=0, plan=None, max_ctx=0):
     T = q.shape[0]
     kc = k_cache.reshape(-1, kv_heads, maps, d).to(F64)
@@ -610,7 +650,7 @@ def masked_attention(q, k_cache, v_cache, tok_req, positions, block_table, page_
             lo = p - p % chunk
         if window > 0:
             lo = max(lo, p - window + 1)
-        js = torch.arange(lo, p + 1)
+        js = torch.cat([torch.arange(min(keep, lo)), torch.arange(lo, p + 1)])
         rows = block_table[r].long()[js // page_size] * page_size + js % page_size
         for h in range(heads):
             g = h // (heads // kv_heads)
@@ -619,6 +659,8 @@ def masked_attention(q, k_cache, v_cache, tok_req, positions, block_table, page_
                 s = (kc[rows, g, m] @ qq[t, h, m]) * scale
                 if r1 is not None:
                     s = s - float(r1[h]) * torch.log1p(float(r2[h]) * (p - js).to(F64))
+                if cap > 0:
+                    s = cap * torch.tanh(s / cap)
                 top = s.max() if sink is None else torch.maximum(s.max(), sink[h].to(F64))
                 e = torch.exp(s - top)
                 total = e.sum() + (torch.exp(sink[h].to(F64) - top) if sink is not None else 0.0)
@@ -699,6 +741,39 @@ def attention_rows(proj, nq, nk, nv, d, dv, out_dtype, k_cache, v_cache, rows, b
     return qk[:, :nq].reshape(T, nq * d).to(out_dtype), values
 
 
+def attention_heads(proj, nq, nk, nv, d, dv, out_dtype, k_cache, v_cache, rows, values_are_keys=False, bias=None,
+                    q_weight=None, k_weight=None, eps=0.0, table=None, rot=0, half=True, positions=None,
+                    temperature=None):
+    T = proj.shape[0]
+    C = (nq + nk) * d + (0 if values_are_keys else nv * dv)
+    y = proj[:, :C].to(F64)
+    if bias is not None:
+        y = y + bias.to(F64)
+    q, k = y[:, :nq * d].reshape(T, nq, d), y[:, nq * d:(nq + nk) * d].reshape(T, nk, d)
+    v = y[:, nq * d:(nq + nk) * d] if values_are_keys else y[:, (nq + nk) * d:]
+    if q_weight is not None:
+        q = q / torch.sqrt((q * q).mean(-1, keepdim=True) + eps) * q_weight.to(F64)
+        k = k / torch.sqrt((k * k).mean(-1, keepdim=True) + eps) * k_weight.to(F64)
+    qk = torch.cat([q, k], dim=1).clone()
+    if table is not None:
+        cs = table[positions.long()].to(F64)
+        cos, sin = cs[:, None, :rot // 2], cs[:, None, rot // 2:]
+        one, other = (slice(0, rot // 2), slice(rot // 2, rot)) if half else (slice(0, rot, 2), slice(1, rot, 2))
+        a, b = qk[..., one].clone(), qk[..., other].clone()
+        qk[..., one] = a * cos - b * sin
+        qk[..., other] = b * cos + a * sin
+    if temperature is not None:
+        coef, every = temperature
+        qk[:, :nq] *= (1 + coef * torch.log(torch.floor((positions.to(F64) + 1) / every) + 1))[:, None, None]
+    if rows is not None:
+        page = k_cache.shape[1]
+        keep = rows >= 0
+        at = rows[keep].long()
+        k_cache[at // page, at % page] = qk[keep, nq:].reshape(-1, nk * d).to(k_cache.dtype)
+        v_cache[at // page, :, at % page] = v[keep].to(v_cache.dtype)
+    return qk[:, :nq].reshape(T, nq * d).to(out_dtype)
+
+
 def mlstm_prepare(proj, heads, key_dim, value_dim, i_column, f_column, i_bias, f_bias, cap, q_scale, reference, q_offsets,
                   slot_ids, num_requests):
     T, nk = proj.shape[0], heads * key_dim
@@ -742,7 +817,8 @@ ALL = ("layer_norm", "layer_norm_act", "embedding_sinusoid", "gated_activation",
        "latent_prepare", "latent_attention", "moe_route", "moe_experts", "moe_combine",
        "scale_", "token_shift", "rms_shift", "moe_route_sigmoid", "lightning_prepare", "lightning_readout",
        "gated_activation_weighted", "attention_prepare", "masked_attention", "state_space_prepare",
-       "state_space_readout", "scaled_sum", "bias_add", "attention_rows", "mlstm_prepare", "mlstm_readout")
+       "state_space_readout", "scaled_sum", "bias_add", "attention_rows", "mlstm_prepare", "mlstm_readout",
+       "attention_heads", "channel_delta_prepare", "gated_linear_prepare", "stream_norms")
 
 
 def install(monkeypatch):
