@@ -1,0 +1,648 @@
+"""The Nogosun design on the GPU: every kernel it brought against the plain torch version of the same operation, and the
+engine against the plain whole-sequence implementation (``plain_nogosun``) in the four families of traces, in float32
+and in bfloat16."""
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+import nogosun_configs as nc
+import plain_nogosun
+import reference_ops
+import traces
+from helpers import make_runner, prompts_for, random_weights, replay
+from lucciola_amd.config.engine_config import EngineConfig
+from lucciola_amd.config.registry import architecture_for
+from lucciola_amd.engine.batch import Plan, StepEntry
+from lucciola_amd.engine.llm_engine import LLMEngine
+from lucciola_amd.engine.loading import _build
+from lucciola_amd.kernels import ops
+from lucciola_amd.sampling.sampler import SamplingParams
+from lucciola_amd.weights.loader import DictSource
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+# A row's error: root mean square of the difference of the logits, means taken off, over that of the plain logits.  In
+# bfloat16 a router's choice between two experts whose scores nearly tie can fall the other way, which changes that row
+# by any amount: the bound is on the median row, on the share of rows over 10 % and on the share of rows that are
+# unrelated.  What a fault of the cache, the state or the batch does wrong shows in many rows, and in float32.
+TOL = {"float32": 6e-5, "bfloat16": 1e-1}
+LENGTHS = {"A": [5, 1, 47, 90, 130], "B": [2, 61, 33, 100], "C": [150, 9, 230, 70]}
+_cache = {}
+
+
+def weights_for(cfg, seed, std=nc.STD):
+    return nc.telling_weights(random_weights(cfg, seed, std=std), seed)
+
+
+def plain_logits(cfg, weights, prompts):
+    w = {k: v.to(torch.float64) for k, v in weights.items()}
+    return {n: plain_nogosun.forward(cfg, w, ids) for n, ids in prompts.items()}
+
+
+def case(key):
+    if key not in _cache:
+        cfg, page, seed = nc.ALL[key]
+        weights = weights_for(cfg, seed)
+        prompts = prompts_for({"vocab_size": cfg["vocab"]}, LENGTHS[key], seed)
+        _cache[key] = (cfg, page, weights, prompts, plain_logits(cfg, weights, prompts))
+    return _cache[key]
+
+
+def row_error(row, ref):
+    diff = row - ref
+    return float((diff - diff.mean()).pow(2).mean().sqrt() / (ref - ref.mean()).pow(2).mean().sqrt())
+
+
+def check_rows(got, prompts, refs, dtype, every=True):
+    errors = []
+    for name, ids in prompts.items():
+        for pos in range(len(ids)):
+            if (name, pos) not in got:
+                assert not every, f"{name} position {pos}: no logits"
+                continue
+            row, ref = got[(name, pos)], refs[name][pos]
+            assert torch.isfinite(row).all(), f"{name} position {pos}: logits are not finite"
+            errors.append((row_error(row, ref), name, pos))
+    tol = TOL[str(dtype).replace("torch.", "")]
+    over = sorted(e for e in errors if e[0] > tol)
+    worst = max(errors)
+    if tol == TOL["bfloat16"]:
+        median = sorted(errors)[len(errors) // 2]
+        assert median[0] <= 0.04, f"the median row's error is {median[0]:.3e}"
+        assert len(over) <= max(1, len(errors) // 10), f"{len(over)} of {len(errors)} rows over {tol:.1e}"
+        unrelated = [e for e in errors if e[0] > 0.6]
+        assert len(unrelated) <= max(1, len(errors) // 50), f"{len(unrelated)} of {len(errors)} rows are unrelated"
+        return worst[0]
+    assert worst[0] <= 3 * tol, f"request {worst[1]} position {worst[2]}: error {worst[0]:.3e} (bound {tol:.1e})"
+    assert len(over) <= max(1, len(errors) // 50), (
+        f"{len(over)} of {len(errors)} rows over {tol:.1e}; first: request {over[0][1]} position {over[0][2]} "
+        f"({over[0][0]:.3e})")
+    return worst[0]
+
+
+def close(got, want, dtype, what, scale=1.0):
+    tol = (4e-6 if dtype == torch.float32 else 1.2e-2) * scale
+    err = float((got.double() - want.double()).abs().max() / want.double().abs().max().clamp_min(1e-9))
+    assert err < tol, f"{what}: relative error {err:.3e}"
+
+
+def request_lists(lengths, slots):
+    q_offsets = torch.tensor([sum(lengths[:i]) for i in range(len(lengths) + 1)], dtype=torch.int32)
+    tok_req = torch.tensor([r for r, n in enumerate(lengths) for _ in range(n)], dtype=torch.int32)
+    return tok_req, q_offsets, torch.tensor(slots, dtype=torch.int32)
+
+
+# ------------------------------------------------------------------ kernels alone
+HEADS_CASES = [
+    # q heads, k heads, d, dv, page, tokens, rot, half, bias, norm, values are keys, temperature
+    (8, 2, 32, 48, 16, 37, 16, True, True, False, False, None),
+    (8, 2, 32, 32, 16, 1, 32, True, True, False, True, None),
+    (9, 3, 10, 7, 4, 5, 6, True, True, True, False, (0.5, 7)),
+    (3, 3, 7, 7, 8, 70, 0, True, True, False, True, None),
+    (16, 4, 128, 128, 16, 300, 64, True, True, True, False, (0.3, 64)),
+    (6, 6, 128, 128, 16, 40, 32, True, True, False, True, None),
+    (4, 2, 48, 64, 16, 33, 0, True, True, True, False, (0.5, 256)),
+    (5, 1, 24, 12, 4, 6, 12, False, False, True, False, (1.2, 1)),
+    (2, 1, 256, 256, 16, 2, 2, True, False, False, True, (0.1, 1000)),
+    (2, 2, 256, 16, 16, 20, 256, True, True, True, False, None),
+    (6, 2, 20, 20, 8, 33, 4, True, True, False, True, None),
+    (4, 4, 16, 16, 8, 9, 16, False, True, True, True, (0.9, 3)),
+]
+
+
+def rotary_table(rot, count=3000):
+    if not rot:
+        return None
+    angle = torch.arange(count, dtype=torch.float64)[:, None] * (
+        300.0 ** (-torch.arange(rot // 2, dtype=torch.float64) * 2 / rot))[None, :]
+    return (torch.cat([torch.cos(angle), torch.sin(angle)], dim=1) * 1.3).float()
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("case_", HEADS_CASES)
+@pytest.mark.parametrize("extra", [5, 8])       # columns behind the heads: with 5, rows begin at odd places
+def test_attention_heads(case_, dtype, extra):
+    """q and the cache rows (and every row that is not a token's: untouched)."""
+    nq, nk, d, dv, page, T, rot, half, bias, norm, keys, temperature = case_
+    g = torch.Generator().manual_seed(nq * 100 + d)
+    C = (nq + nk) * d + (0 if keys else nk * dv)
+    proj = torch.randn(T, C + extra, generator=g) * 2
+    pages = T // page + 4
+    places = torch.randperm(pages * page, generator=g)[:T].to(torch.int32)
+    places[T // 2] = -1 if T > 2 else places[T // 2]
+    positions = torch.randint(0, 3000, (T,), generator=g).to(torch.int32)
+    tensors = dict(bias=torch.randn(C, generator=g) if bias else None,
+                   q_weight=1 + 0.3 * torch.randn(d, generator=g) if norm else None,
+                   k_weight=1 + 0.3 * torch.randn(d, generator=g) if norm else None, table=rotary_table(rot),
+                   positions=positions)
+    outs = []
+    for o, where in ((reference_ops, "cpu"), (ops, DEV)):
+        def on(t):
+            return None if t is None else t.clone().to(where)
+        kc = torch.full((pages, page, nk * d), 7.0, dtype=dtype, device=where)
+        v_cache = torch.full((pages, nk * dv, page), 7.0, dtype=dtype, device=where)
+        q = o.attention_heads(on(proj), nq, nk, nk, d, dv, dtype, kc, v_cache, on(places), values_are_keys=keys, eps=1e-5,
+                              rot=rot, half=half, temperature=temperature, **{k: on(v) for k, v in tensors.items()})
+        outs.append([t.cpu() for t in (q, kc, v_cache)])
+    for got, want, what in zip(outs[1], outs[0], ("q", "key rows", "value rows")):
+        close(got, want, dtype, what)
+
+
+@pytest.mark.parametrize("position,every", [(0, 1), (5, 7), (6, 7), (7, 7), (254, 256), (255, 256), (256, 256), (2559, 10),
+                                            (2558, 10), (99999, 100000), (100000, 100000)])
+def test_the_temperature_changes_where_it_should(position, every):
+    """The step of the query's factor lies between positions n every - 2 and n every - 1."""
+    d = 8
+    proj = torch.ones(1, 3 * d, device=DEV)
+    caches = (torch.zeros(1, 16, d, device=DEV), torch.zeros(1, d, 16, device=DEV))
+    q = ops.attention_heads(proj, 1, 1, 1, d, d, torch.float32, *caches, None,
+                            positions=torch.tensor([position], dtype=torch.int32, device=DEV), temperature=(0.5, every))
+    want = 1 + 0.5 * float(np.log((position + 1) // every + 1))
+    assert float((q - want).abs().max()) < 2e-6 * want
+
+
+MASK_CASES = [
+    # heads, kv heads, d, dv, page, window, keep, cap, sink, gate
+    (8, 2, 32, 32, 16, 40, 6, 0.0, None, False),
+    (6, 6, 128, 128, 16, 33, 17, 0.0, None, False),
+    (4, 2, 48, 64, 16, 0, 0, 30.0, 0.0, True),
+    (4, 1, 16, 32, 32, 1, 1, 2.0, 0.7, False),
+    (16, 2, 64, 64, 16, 16, 70, 5.0, 0.0, True),
+    (3, 3, 10, 10, 8, 9, 3, 1.5, 0.0, False),
+    (2, 1, 256, 256, 4, 30, 5, 0.0, None, True),
+    (32, 1, 64, 16, 16, 100, 3, 8.0, None, False),
+    (5, 5, 80, 80, 48, 7, 20, 0.0, None, False),
+]
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("case_", MASK_CASES)
+def test_masked_attention_with_kept_keys_and_caps(case_, dtype):
+    """Two requests, portions and lone tokens, on every kernel that takes the sizes; the pages between the kept ones and
+    the window hold infinities: they must not be read."""
+    heads, kv, d, dv, page, window, keep, cap, sink_value, gated = case_
+    g = torch.Generator().manual_seed(heads + d)
+    lengths, news = (300, 170), (50, 1)
+    width = max(lengths) // page + 2
+    pages = 2 * width + 3
+    tables = torch.randperm(pages, generator=g)[:2 * width].to(torch.int32).view(2, width)
+    k_cache = torch.randn(pages, page, kv * d, generator=g) * (2.0 / d ** 0.5)
+    v_cache = torch.randn(pages, kv * dv, page, generator=g)
+    for r, (length, new) in enumerate(zip(lengths, news)):
+        if window:
+            first = max(0, length - new - window + 1) // page       # the page of the first key that anyone sees
+            for i in range(-(-keep // page), first):
+                k_cache[tables[r, i]] = float("inf")
+                v_cache[tables[r, i]] = float("inf")
+    k_cache, v_cache = k_cache.to(dtype), v_cache.to(dtype)
+    q = (torch.randn(sum(news), heads * d, generator=g) * 3).to(dtype)
+    gate = torch.randn(sum(news), heads * dv + 3, generator=g)
+    positions = torch.tensor([p for length, new in zip(lengths, news) for p in range(length - new, length)], dtype=torch.int32)
+    tok_req = torch.tensor([r for r, new in enumerate(news) for _ in range(new)], dtype=torch.int32)
+    sink = None if sink_value is None else torch.full((heads,), sink_value)
+
+    def run(o, where, **more):
+        def on(t):
+            return None if t is None else t.to(where)
+        return o.masked_attention(on(q), on(k_cache), on(v_cache), on(tok_req), on(positions), on(tables), page, heads, kv, 1,
+                                  d, dv, 0.5, window=window, keep=keep if window else 0, cap=cap, sink=on(sink),
+                                  gate=on(gate) if gated else None, gate_column=3, **more).cpu()
+    want = run(reference_ops, "cpu")
+    close(run(ops, DEV), want, dtype, "general kernel", 2.0)
+    if not ops.masked_attention_on_matrix_cores(dtype, d, dv, page, 1):
+        return
+    for cut in (16, 5, 1):
+        tiles = [[i, min(cut, news[0] - i), 0, lengths[0] - news[0] + i] for i in range(0, news[0], cut)]
+        tiles.append([news[0], 1, 1, lengths[1] - 1])
+        plan = Plan({"tiles": torch.tensor(tiles, dtype=torch.int32, device=DEV)},
+                    {"any_portion": cut > 1, "any_lone": True})
+        for staged in (True, False):
+            before = ops.masked_attention_staged(staged)
+            try:
+                close(run(ops, DEV, plan=plan), want, dtype, f"matrix cores, tiles of {cut}, staged {staged}", 2.0)
+            finally:
+                ops.masked_attention_staged(before)
+
+
+@pytest.mark.parametrize("splits", [1, 2, 5, 16])
+def test_lone_tokens_over_several_workgroups_with_kept_keys(splits):
+    heads, kv, d, dv, page, length, window, keep = 8, 2, 64, 32, 16, 1500, 1100, 200
+    g = torch.Generator().manual_seed(3)
+    width = length // page + 1
+    table = torch.randperm(width + 2, generator=g)[:width].to(torch.int32).view(1, -1)
+    k_cache = (torch.randn(width + 2, page, kv * d, generator=g) * 0.3).to(torch.bfloat16)
+    v_cache = torch.randn(width + 2, kv * dv, page, generator=g).to(torch.bfloat16)
+    q = (torch.randn(1, heads * d, generator=g) * 2).to(torch.bfloat16)
+    args = (torch.zeros(1, dtype=torch.int32), torch.tensor([length - 1], dtype=torch.int32), table)
+    more = dict(window=window, keep=keep, cap=4.0, sink=torch.zeros(heads))
+    want = reference_ops.masked_attention(q, k_cache, v_cache, *args, page, heads, kv, 1, d, dv, 1.0, **more)
+    plan = Plan({"tiles": torch.tensor([[0, 1, 0, length - 1]], dtype=torch.int32, device=DEV)},
+                {"any_portion": False, "any_lone": True})
+    before = ops.masked_attention_force_splits(splits)
+    try:
+        more["sink"] = more["sink"].to(DEV)
+        got = ops.masked_attention(q.to(DEV), k_cache.to(DEV), v_cache.to(DEV), *(t.to(DEV) for t in args), page, heads, kv, 1,
+                                   d, dv, 1.0, plan=plan, max_ctx=length, **more)
+    finally:
+        ops.masked_attention_force_splits(before)
+    close(got.cpu(), want, torch.bfloat16, f"{splits} workgroups", 2.0)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("window,keep", [(1, 1), (16, 15), (16, 16), (16, 17), (17, 3), (40, 33), (100, 2), (15, 0), (64, 300)])
+def test_one_key_carries_the_weight_at_a_windows_and_the_kept_ones_edges(dtype, window, keep):
+    """Among hundreds of keys one has a score that stands out and a value of its own: a query sees it exactly when it is
+    not ahead and fewer than ``window`` tokens lie between them or it is one of the first ``keep``; in prompts, in portions
+    that begin anywhere and in lone tokens, at page borders and at a sequence's start, on all attention kernels."""
+    heads, kv, d, dv, page, length = 4, 2, 32, 32, 16, 260
+    g = torch.Generator().manual_seed(window)
+    table = torch.randperm(length // page + 3, generator=g)[:length // page + 1].to(torch.int32).view(1, -1)
+    places = torch.tensor([int(table[0, p // page]) * page + p % page for p in range(length)], device=DEV)
+    k_cache = torch.zeros(length // page + 3, page, kv * d, dtype=dtype, device=DEV)
+    v_cache = torch.zeros(length // page + 3, kv * dv, page, dtype=dtype, device=DEV)
+    q = torch.ones(length, heads * d, dtype=dtype, device=DEV)
+    for marked in sorted({0, 1, 15, 16, 31, 100, 111, 112, 200} | {m for m in (keep - 1, keep, keep + 1) if 0 <= m < length}):
+        k = torch.zeros(length, kv * d, dtype=dtype, device=DEV)
+        v = torch.full((length, kv * dv), -1.0, dtype=dtype, device=DEV)
+        k[marked], v[marked] = 1.0, 5.0
+        k_cache.view(-1, kv * d)[places], v_cache[places // page, :, places % page] = k, v
+        edge = marked + window
+        lone_rows = sorted({p for p in (marked - 1, marked, marked + 1, edge - 1, edge, edge + 1, length - 1) if 0 <= p < length})
+        for lone in (False, True):
+            rows = lone_rows if lone else list(range(length))
+            plans = [None]
+            if ops.masked_attention_on_matrix_cores(dtype, d, dv, page, 1):
+                for cut in ((1,) if lone else (16, 7, 2)):      # tiles of so many tokens
+                    tiles = [[i, min(cut, len(rows) - i), 0, rows[i]] for i in range(0, len(rows), cut)]
+                    plans.append(Plan({"tiles": torch.tensor(tiles, dtype=torch.int32, device=DEV)},
+                                      {"any_portion": not lone, "any_lone": any(t[1] == 1 for t in tiles)}))
+            want = []
+            for p in rows:
+                seen = sum(1 for j in range(p + 1) if p - j < window or j < keep)
+                sees = marked <= p and (p - marked < window or marked < keep)
+                top, others = (float(np.exp(32.0)) if sees else 0.0), seen - int(sees)
+                want.append((5.0 * top - others) / (top + others))
+            want = torch.tensor(want)
+            for plan in plans:
+                out = ops.masked_attention(q[:len(rows)].contiguous(), k_cache, v_cache,
+                                           torch.zeros(len(rows), dtype=torch.int32, device=DEV),
+                                           torch.tensor(rows, dtype=torch.int32, device=DEV), table.to(DEV), page, heads, kv,
+                                           1, d, dv, 1.0, window=window, keep=keep, plan=plan).float().cpu()
+                wrong = ((out[:, [0, 3 * dv]] - want[:, None]).abs().amax(1) > 5e-2).nonzero().flatten().tolist()
+                assert not wrong, (f"key {marked}, query {rows[wrong[0]]} ({'lone' if lone else 'prompt'}, "
+                                   f"{'general' if plan is None else 'matrix cores'}): {out[wrong[0], 0]:.3f}, "
+                                   f"expected {want[wrong[0]]:.3f}")
+
+
+DELTA_CASES = [
+    # heads, kv heads, dk, dv, taps, lengths of two steps
+    (4, 2, 32, 40, 4, [70, 1, 129, 2]),
+    (3, 3, 7, 5, 1, [3, 200, 1, 64]),
+    (2, 1, 128, 128, 4, [65, 130, 1, 33]),
+    (6, 2, 16, 16, 2, [1, 1, 1, 1]),
+    (5, 5, 64, 31, 9, [5, 12, 2, 38]),
+    (2, 2, 256, 8, 3, [1, 1, 40, 1]),
+]
+
+
+@pytest.mark.parametrize("case_", DELTA_CASES)
+def test_channel_delta_kernels(case_):
+    """Three steps in a row over the same slots: the scan's inputs, the tails, the scan and the read-out against their plain
+    versions, and the slots of other requests untouched."""
+    heads, kv, dk, dv, taps, lengths = case_
+    g = torch.Generator().manual_seed(dk)
+    C, nk, nv = 2 * kv * dk + heads * dv, heads * dk, heads * dv
+    conv = torch.randn(C, taps, generator=g)
+    rate_log, rate_bias = torch.randn(heads, generator=g) - 1, torch.randn(nk, generator=g)
+    weight = 1 + 0.3 * torch.randn(dv, generator=g)
+    slots = [4, 0, 5, 2]
+    states = {where: (torch.zeros(7, heads, dv, dk, device=where), torch.zeros(7, taps - 1, C, device=where))
+              for where in ("cpu", DEV)}
+    for step, new in enumerate((lengths, lengths[::-1], [1, 2, 1, 1])):
+        lists = request_lists(new, slots)
+        proj = torch.randn(sum(new), C + heads + 3, generator=g)
+        rates = torch.randn(sum(new), nk + nv + 2, generator=g) * 2
+        outs = []
+        for o, where in ((reference_ops, "cpu"), (ops, DEV)):
+            state, tail = states[where]
+            tok_req, q_offsets, slot_ids = (t.to(where) for t in lists)
+            pj, rt = proj.to(where), rates.to(where)
+            coef, v = o.channel_delta_prepare(pj, C + 2, rt, 1, tail, conv.to(where), rate_log.to(where), rate_bias.to(where),
+                                              heads, kv, dk, dv, taps, 1e-6, tok_req, q_offsets, slot_ids)
+            o.conv_tail_update(pj, tail, C, taps, q_offsets, slot_ids, len(new))
+            y = o.delta_scan(coef, v, state, q_offsets, slot_ids, len(new), heads, dk, dv)
+            z = o.head_gate_norm(y, rt, nk + 1, weight.to(where), False, 1e-5, "sigmoid", heads, dv, torch.float32)
+            outs.append([t.cpu() for t in (coef[0], coef[1], coef[2], coef[3], coef[4], v, tail, y, state, z)])
+        for got, want, what in zip(outs[1], outs[0], ("decay", "probe", "removal", "write", "read", "values", "tails", "scan",
+                                                      "state", "read-out")):
+            if want.numel():
+                close(got, want, torch.float32, f"step {step}: {what}", 40.0 if what == "read-out" else 8.0)
+        for slot in (1, 3, 6):
+            assert float(states[DEV][0][slot].abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("heads,dk,dv,tau", [(6, 32, 64, 16.0), (3, 7, 5, 1.0), (1, 128, 128, 4.0), (2, 256, 8, 100.0)])
+def test_gated_linear_kernels(heads, dk, dv, tau):
+    g = torch.Generator().manual_seed(dk)
+    nk, nv = heads * dk, heads * dv
+    bias, weight = torch.randn(nk, generator=g), 1 + 0.3 * torch.randn(dv, generator=g)
+    slots = [4, 0, 5]
+    states = {where: torch.zeros(7, heads, dv, dk, device=where) for where in ("cpu", DEV)}
+    for step, new in enumerate(([70, 1, 33], [2, 100, 1], [1, 1, 1])):
+        _, *lists = request_lists(new, slots)
+        proj = torch.randn(sum(new), 2 * nk + 2 * nv + 1, generator=g)
+        rates = torch.randn(sum(new), nk + 3, generator=g) * 20         # both ends of the sigmoid
+        outs = []
+        for o, where in ((reference_ops, "cpu"), (ops, DEV)):
+            q_offsets, slot_ids = (t.to(where) for t in lists)
+            pj = proj.to(where)
+            coef, v = o.gated_linear_prepare(pj, rates.to(where), 2, bias.to(where), 1 / tau, dk ** -0.5, heads, dk, dv)
+            y = o.delta_scan(coef, v, states[where], q_offsets, slot_ids, len(new), heads, dk, dv)
+            z = o.head_gate_norm(y, pj, 2 * nk + nv, weight.to(where), False, 1e-5, "silu", heads, dv, torch.float32)
+            outs.append([t.cpu() for t in (coef[0], coef[1], coef[2], v, y, states[where], z)])
+        for got, want, what in zip(outs[1], outs[0], ("decay", "write", "read", "values", "scan", "state", "read-out")):
+            close(got, want, torch.float32, f"step {step}: {what}", 40.0 if what == "read-out" else 8.0)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("T,n,K", [(1, 256, 384), (7, 50, 30), (3, 640, 128), (16, 2048, 2048), (70, 4096, 256), (33, 128, 2048),
+                                   (5, 6000, 128), (2, 8200, 128), (9, 1000, 512)])
+def test_branches_join_the_stream_and_are_normed_twice(dtype, T, n, K):
+    """Products (cut along K or not), rows of experts and tensors, each with a factor, at all rows and at picked ones."""
+    g = torch.Generator().manual_seed(n)
+    h = torch.randn(T, n, generator=g)
+    w1, w2 = (1 + 0.3 * torch.randn(n, generator=g) for _ in range(2))
+    x = torch.randn(T, K, generator=g).to(dtype)
+    w = (torch.randn(n, K, generator=g) / K ** 0.5).to(dtype)
+    other = torch.randn(T, n, generator=g)
+    top, experts = 3, 5
+    y = torch.randn(T * top, n, generator=g)
+    logits = torch.randn(T, experts, generator=g).to(DEV)
+    rows = torch.tensor([T - 1, 0, T // 2], dtype=torch.int32)
+    routing = ops.moe_route(logits, top, renormalise=False)
+    mixed = (routing.weights.cpu().double()[:, :, None] * y.double()[routing.entry_row.cpu().view(T, top).long()]).sum(1)
+    product = x.double() @ w.double().T
+    for branches, total in (
+            (((ops.gemm(x.to(DEV), w.to(DEV), dtype, defer=True), 1.2), (other.to(DEV), -0.9),
+              (ops.RoutedRows(y.to(DEV), routing, dtype), 1.0)), 1.2 * product - 0.9 * other.double() + mixed),
+            (((ops.gemm(x.to(DEV), w.to(DEV), dtype), 0.5),), 0.5 * product),
+            (((other.to(dtype).to(DEV), 2.0), (ops.RoutedRows(y.to(DEV), routing, dtype), 3.0)),
+             2.0 * other.to(dtype).double() + 3.0 * mixed)):
+        v = h.double() + total
+        normed = v / torch.sqrt((v * v).mean(-1, keepdim=True) + 1e-5)
+        stream = h.clone().to(DEV)
+        got = ops.stream_norms(stream, ops.SummedBranches(branches), (w1.to(DEV), w2.to(DEV)), 1e-5, dtype)
+        close(got[0].cpu(), normed * w1.double(), dtype, "first")
+        close(got[1].cpu(), normed * w2.double(), dtype, "second")
+        close(stream.cpu(), v, torch.float32 if dtype == torch.float32 else dtype, "stream", 2.0)
+        stream = h.clone().to(DEV)
+        picked = ops.rmsnorm(stream, ops.SummedBranches(branches), w2.to(DEV), 1e-5, dtype, rows=rows.to(DEV))
+        close(picked.cpu(), (normed * w2.double())[rows.long()], dtype, "picked rows")
+        assert torch.equal(stream.cpu(), h)
+        close(ops.value(ops.SummedBranches(branches)).cpu(), total, dtype, "value", 2.0)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("T,H,I,E,top", [(1, 64, 20, 5, 2), (40, 128, 96, 8, 4), (300, 256, 128, 4, 1), (900, 128, 256, 4, 2)])
+def test_experts_with_the_exact_gelu(dtype, T, H, I, E, top):
+    from lucciola_amd.parts import BuildContext
+    from lucciola_amd.parts.feed_forward import RoutedMLP
+    g = torch.Generator().manual_seed(T)
+    part = RoutedMLP(H, I, E, top, activation="gelu", renormalise=False)
+    tensors = {n: (torch.randn(tuple(d.shape), generator=g) * (3.0 if n == "router" else 2.0) / d.shape[1] ** 0.5).to(torch.bfloat16)
+               for n, d in part.declare().items()}
+    x = torch.randn(T, H, generator=g).to(dtype)
+    part.bind({n: t.to(dtype).to(DEV) for n, t in tensors.items()}, BuildContext(dtype=dtype, device=torch.device(DEV)))
+    w = {"x." + n.replace("experts.", "e"): t.double() for n, t in tensors.items()}
+    want = plain_nogosun.experts(x.double(), w, "x.", {"router": {"experts": E, "top": top}})
+    close(part.forward(x.to(DEV)).cpu(), want, dtype, "experts", 2.0)
+
+
+# ------------------------------------------------------------------ the engine
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("key", ["A", "B", "C"])
+@pytest.mark.parametrize("family", ["whole", "tail", "chunked", "mixed"])
+def test_replay_families(dtype, key, family):
+    cfg, page, weights, prompts, refs = case(key)
+    steps = {"whole": traces.whole, "tail": traces.tail_decode, "chunked": traces.chunked,
+             "mixed": traces.mixed}[family](prompts)
+    blocks = traces.max_live_tokens(steps, page) // page
+    runner = make_runner(cfg, weights, page, blocks, dtype, DEV)
+    check_rows(replay(runner, steps), prompts, refs, dtype)
+    assert not runner.cache.requests
+    for g in runner.cache.groups:
+        assert g.pool.num_free() == blocks
+
+
+ATT = dict(heads=4, kv_heads=2, dim=16, scale=0.3)
+LEFT, RIGHT = (4, 2, 12, 8, 0.3, 8.0, 0.5, 16), (2, 8, 16, 4.0)
+MECHANISMS = {
+    "attention alone": [nc.layer(nc.attention(**ATT))],
+    "attention in a window": [nc.layer(nc.attention(**ATT, window=13))],
+    "a window of one token beside the first": [nc.layer(nc.attention(3, 1, 8, 0.3, 1, 1, rot_dims=8))],
+    "more kept tokens than the window": [nc.layer(nc.attention(2, 2, 8, 0.3, 5, 19))],
+    "kept tokens over a page's edge": [nc.layer(nc.attention(2, 1, 32, 0.3, 16, 9, rot_dims=16))],
+    "rotation of some entries, stretched": [nc.layer(nc.attention(2, 1, 16, 0.3, 9, 2, 6, 50.0, (4.0, 40, 8.0, 1.0)))],
+    "rotation of all entries": [nc.layer(nc.attention(2, 1, 16, 0.3, 30, 3, rot_dims=16, base=9000.0))],
+    "two layers of the same tensors": [nc.layer(nc.attention(2, 1, 8, 0.3, 9, 2, rot_dims=4))] * 1,
+    "capped attention mostly": [nc.layer(nc.parallel(LEFT, RIGHT, 1.5, 0.1))],
+    "a low cap and a temperature that grows with every token": [
+        nc.layer(nc.parallel((2, 1, 8, 20, 0.5, 0.8, 1.5, 1), RIGHT, 1.0, 0.2))],
+    "gated linear attention mostly": [nc.layer(nc.parallel(LEFT, RIGHT, 0.1, -1.5))],
+    "slow forgetting": [nc.layer(nc.parallel(LEFT, (4, 16, 8, 200.0), 0.2, 1.0))],
+    "the delta rule alone": [nc.layer(nc.channel_delta(4, 4, 16, 8, 4))],
+    "the delta rule with shared keys": [nc.layer(nc.channel_delta(6, 2, 8, 12, 2))],
+    "the delta rule with one tap": [nc.layer(nc.channel_delta(2, 1, 5, 7, 1))],
+    "all experts": [nc.layer(nc.channel_delta(2, 2, 4, 4, 3), 12, 4, 4)],
+    "one expert of many": [nc.layer(nc.attention(**ATT, window=6, keep=2), 16, 9, 1)],
+}
+MECHANISMS["two layers of the same tensors"].append(nc.borrows(MECHANISMS["two layers of the same tensors"], 0))
+for base in ("the delta rule alone", "capped attention mostly"):
+    MECHANISMS["borrowed: " + base] = MECHANISMS[base] + [nc.borrows(MECHANISMS[base], 0)]
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", sorted(MECHANISMS))
+def test_each_mechanism(name, dtype):
+    cfg = {"architecture": "Nogosun", "vocab": 90, "width": 48, "norm": {"eps": 1e-5}, "embedding": {"scale": 4.0},
+           "layers": MECHANISMS[name]}
+    weights = weights_for(cfg, 5, std=0.09)
+    prompts = prompts_for({"vocab_size": 90}, [37, 4, 60], 2)
+    refs = plain_logits(cfg, weights, prompts)
+    steps = traces.chunked(prompts, sizes=(7, 2, 16, 1, 1, 3, 30))
+    runner = make_runner(cfg, weights, 8, traces.max_live_tokens(steps, 8) // 8, dtype, DEV)
+    check_rows(replay(runner, steps), prompts, refs, dtype)
+
+
+def test_float32_logits_do_not_depend_on_the_cut():
+    """The same bits whole, in portions and token by token: every sum's order follows from the token alone."""
+    for key in ("A", "B"):
+        cfg, page, weights, _, _ = case(key)
+        prompts = prompts_for({"vocab_size": cfg["vocab"]}, [75, 40], 3)
+        runs = []
+        for steps in (traces.whole(prompts), traces.chunked(prompts), traces.tail_decode(prompts, tail=30),
+                      traces.mixed(prompts)):
+            runs.append(replay(make_runner(cfg, weights, page, 80, "float32", DEV), steps))
+        for other in runs[1:]:
+            for at, row in runs[0].items():
+                same = torch.equal(row, other[at])
+                assert same, f"{key} {at}: the bits differ between two cuts"
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("key", ["A", "B", "C"])
+def test_a_batch_of_unequal_requests_against_each_alone(key, dtype):
+    cfg, page, weights, prompts, refs = case(key)
+    names = list(prompts)[:4]
+    alone = {}
+    for n in names:
+        alone.update(replay(make_runner(cfg, weights, page, 64, dtype, DEV), traces.whole({n: prompts[n]})))
+    runner = make_runner(cfg, weights, page, 160, dtype, DEV)
+    cut = {n: max(1, len(prompts[n]) - 3) for n in names}
+    rest = {n: prompts[n][cut[n]:] for n in names}
+    steps = [([(n, prompts[n][:cut[n]], list(range(cut[n]))) for n in names], [n for n in names if not rest[n]])]
+    for k in range(max(len(r) for r in rest.values())):
+        steps.append(([(n, [rest[n][k]], [0]) for n in names if k < len(rest[n])],
+                      [n for n in names if k == len(rest[n]) - 1]))
+    together = replay(runner, steps)
+    assert sorted(together) == sorted(alone)
+    for at, row in alone.items():
+        if dtype == "float32":
+            same = torch.equal(row, together[at])
+            assert same, f"{at}: the bits differ between alone and in a batch"
+    if dtype == "bfloat16":         # a router's close call may fall the other way
+        errors = sorted(row_error(together[at], row) for at, row in alone.items())
+        assert errors[len(errors) // 2] < 4e-2 and errors[int(0.9 * len(errors))] < 0.1
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("seed", range(12))
+def test_random_configurations(seed, dtype):
+    """Configurations drawn at random, requests in mixed steps with so few pages and slots that they are used
+    again, against the plain implementation."""
+    cfg, page = nc.random_configuration(seed)
+    weights = weights_for(cfg, 100 + seed)
+    prompts = prompts_for({"vocab_size": cfg["vocab"]}, [3, 120, 41, 77, 1, 150], seed)
+    refs = plain_logits(cfg, weights, prompts)
+    steps = traces.mixed(prompts, seed=seed)
+    runner = make_runner(cfg, weights, page, traces.max_live_tokens(steps, page) // page, dtype, DEV)
+    check_rows(replay(runner, steps), prompts, refs, dtype)
+    assert not runner.cache.requests
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("key", ["A", "C"])
+def test_long_decoding_past_windows_with_used_pages_and_slots(dtype, key):
+    """Two slots and few pages: a request decodes token by token until its windows have passed over what it decoded,
+    while others come and go in the pages and slots that earlier ones gave back."""
+    cfg, page, weights, _, _ = case(key)
+    prompts = prompts_for({"vocab_size": cfg["vocab"]}, [150, 30, 26, 41], 9)
+    refs = plain_logits(cfg, weights, prompts)
+    names = list(prompts)
+    long_ids = prompts[names[0]]
+    steps = [([(names[1], prompts[names[1]], [29])], [names[1]]), ([(names[0], long_ids[:20], list(range(20)))], [])]
+    others = [names[2], names[3]]
+    fed = {n: 0 for n in others}
+    for i in range(20, 150):
+        entries, end = [(names[0], [long_ids[i]], [0])], []
+        live = next((n for n in others if fed[n] < len(prompts[n])), None)
+        if live is not None and i % 2:
+            n = min(5, len(prompts[live]) - fed[live])
+            entries.append((live, prompts[live][fed[live]:fed[live] + n], list(range(n))))
+            fed[live] += n
+            if fed[live] == len(prompts[live]):
+                end.append(live)
+        if i == 149:
+            end.append(names[0])
+        steps.append((entries, end))
+    runner = make_runner(cfg, weights, page, traces.max_live_tokens(steps, page) // page, dtype, DEV, max_seqs=2)
+    check_rows(replay(runner, steps), prompts, refs, dtype, every=False)
+    assert not runner.cache.requests
+
+
+def test_replayed_decode_steps_equal_eager_ones():
+    """Steps of single tokens replayed from a HIP graph (states updated in place), with eager portions in between, against a runner that launches every step's kernels."""
+    cfg, page, weights, prompts, _ = case("C")
+    names = list(prompts)[:3]
+    runs = []
+    for graphs in (True, False):
+        runner = make_runner(cfg, weights, page, 80, "bfloat16", DEV)
+        assert runner.use_graphs
+        runner.use_graphs = graphs
+        out = []
+        for n in names:
+            out.append(runner.step([StepEntry(n, prompts[n][:9], [8])]).cpu())
+        for k in range(9, 40):
+            live = [n for n in names if k < len(prompts[n])]
+            out.append(runner.step([StepEntry(n, [prompts[n][k]], [0]) for n in live]).cpu())
+            if k == 20:
+                runner.step([StepEntry("other", prompts[names[0]][:30], [29])])
+                runner.finish("other")
+        assert (runner.graph_replays > 20) == graphs
+        runs.append(out)
+    for a, b in zip(*runs):
+        assert torch.equal(a, b)
+
+
+@pytest.mark.parametrize("key", ["A", "B", "C"])
+def test_greedy_generation_through_the_engine(key):
+    cfg, page, seed = nc.ALL[key]
+    weights = weights_for(cfg, seed, std=0.15)
+    arch = architecture_for(cfg)
+    config = arch.read_config(cfg)
+    w64 = {k: v.to(torch.float64) for k, v in weights.items()}
+    model = _build(arch.model_spec(config), DictSource(weights), "float32", DEV)
+    engine = LLMEngine(model, config, EngineConfig(dtype="float32", block_size=page, max_blocks=60, max_seqs=3,
+                                                   max_tokens_per_step=24, device=DEV))
+    prompts = list(prompts_for({"vocab_size": cfg["vocab"]}, [4, 33, 57, 9], seed + 1).values())
+    got = engine.generate(prompts, SamplingParams(max_new_tokens=8))
+    for p, tokens in zip(prompts, got):
+        assert len(tokens) == 8
+        ids = list(p)
+        for t in tokens:        # every generated token is the plain form's argmax, or a near tie with it
+            logits = plain_nogosun.forward(cfg, w64, ids)[-1]
+            best = int(torch.argmax(logits))
+            assert t == best or float(logits[best] - logits[t]) < 1e-4 * float(logits.abs().max()), (ids, t, best)
+            ids.append(t)
+    engine.runner.cache.check()
+    assert not engine.runner.cache.requests
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_run_program(tmp_path, dtype):
+    """A model folder made from a configuration and a seed, replayed by ``bin/trace_run``: the architecture is found by
+    config.json alone, and the pool is as small as the live requests allow."""
+    from lucciola_amd.weights.random_init import write_model_folder
+    from lucciola_amd.weights.safetensors_io import SafetensorsFile
+    cfg, page, seed = nc.ALL["B"]
+    folder = write_model_folder(str(tmp_path / "model"), dict(cfg, initializer_range=nc.STD), seed)
+    with SafetensorsFile(os.path.join(folder, "model.safetensors")) as f:
+        weights = {n: f.get(n).clone() for n in f.names()}
+    prompts = prompts_for({"vocab_size": cfg["vocab"]}, [70, 33, 50, 3, 61], seed)
+    steps = traces.mixed(prompts, seed=3)
+    lines, index, fed = [], {}, {}
+    for i, (entries, end) in enumerate(steps):
+        lines.append(json.dumps({"step": i, "end": end, "entries": [{"id": n, "tokens": t, "want": w} for n, t, w in entries]}))
+        rows = []
+        for n, t, w in entries:
+            rows += [(n, fed.get(n, 0) + k) for k in w]
+            fed[n] = fed.get(n, 0) + len(t)
+        index[i] = rows
+    out = tmp_path / "out"
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    proc = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", folder, "--dtype", dtype,
+                           "--out", str(out), "--max-tokens", str(traces.max_live_tokens(steps, 64))],
+                          input="\n".join(lines) + "\n", text=True, capture_output=True, timeout=600)
+    assert proc.returncode == 0, proc.stderr[-2000:]
+    assert proc.stdout.split() == [x for i in range(len(steps)) for x in ("done", str(i))]
+    got = {}
+    for i, rows in index.items():
+        data = np.fromfile(out / f"{i}.f32", dtype="<f4").reshape(len(rows), cfg["vocab"])
+        for r, key in enumerate(rows):
+            got[key] = torch.from_numpy(data[r].astype("float64"))
+    check_rows(got, prompts, plain_logits(cfg, weights, prompts), dtype)
