@@ -450,6 +450,31 @@ def vasanex_design_config(name, routed=False):
             "embedding": {"scale": 2.0}, "initializer_range": 0.02, "layers": layers}
 
 
+def nogosun_design_config(name, routed=True):
+    """The Nogosun decoder at the same width, heads, head size, feed-forward width, vocabulary and depth: two mixers side
+    by side (attention with normed heads, a query temperature, capped scores and an output gate, heads of 128 over heads
+    / 4 key/value heads, beside gated linear attention of as many heads of 128 x 128), attention whose values are its
+    keys (heads of 128 over heads / 4, half of each head rotated, window 4,096 beside 4 kept tokens), the delta rule with
+    a decay per channel (heads of 128 x 128 over heads / 4 query/key heads, four taps), and the attention layer's
+    tensors once more; low-rank matrices of a head's size (the delta rule's) and of 16 (the other's).  Every layer has
+    two-matrix experts, 4 of 32 of ff / 4."""
+    width, heads, ff = DESIGN_SIZES[name]
+    kv = max(1, heads // 4)
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 32, "top": 4}}
+    both = {"left": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+                     "q_temp": {"coef": 0.3, "every": 1024}},
+            "right": {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0}, "left_scale": 1.1, "right_scale": 0.9}
+    attention = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                 "mask": {"size": 4096, "keep_first": 4},
+                 "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+    delta = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "conv": 4}
+    layers = [{"type": "parallel", "mixer": both, "mlp": moe}, {"type": "attention", "mixer": attention, "mlp": moe},
+              {"type": "channel_delta", "mixer": delta, "mlp": moe},
+              {"type": "attention", "mixer": attention, "mlp": moe, "weights_of": 1}]
+    return {"architecture": "Nogosun", "vocab": DESIGN_VOCAB, "width": width, "norm": {"eps": 1e-6},
+            "embedding": {"scale": 2.0}, "initializer_range": 0.02, "layers": layers}
+
+
 def design_run(cfg, dtype, dev, block_size, prompt, batches, context, steps):
     """Prompt and decode throughput of one configuration through the runner's own step."""
     import torch
@@ -532,11 +557,12 @@ def designs_workload(args, dev):
                 results[key] = design_run(pubodra, dtype, dev, args.block_size, args.prefill_tokens, batches,
                                           args.design_context, args.steps)
                 say(f"{key}: {results[key]}")
-        for model in ("larupel", "larupel_dense", "kikunex", "kikunex_dense", "rununex", "rununex_dense", "vasanex"):
+        for model in ("larupel", "larupel_dense", "kikunex", "kikunex_dense", "rununex", "rununex_dense", "vasanex",
+                      "nogosun"):
             if model in wanted:
                 key = f"{name}/{model}"
                 make = {"l": larupel_design_config, "k": kikunex_design_config, "r": rununex_design_config,
-                        "v": vasanex_design_config}[model[0]]
+                        "v": vasanex_design_config, "n": nogosun_design_config}[model[0]]
                 results[key] = design_run(make(name, routed="dense" not in model), dtype, dev,
                                           args.block_size, args.prefill_tokens, batches, args.design_context, args.steps)
                 say(f"{key}: {results[key]}")
@@ -588,7 +614,7 @@ def main() -> int:
     ap.add_argument("--design-batches", default="8,64", help="designs: decode batch sizes")
     ap.add_argument("--design-models", default="qwen3,pubodra_dense,pubodra_routed,larupel",
                     help="designs: which of qwen3, pubodra_dense, pubodra_routed, larupel, larupel_dense, kikunex, kikunex_dense, "
-                         "rununex, rununex_dense, vasanex")
+                         "rununex, rununex_dense, vasanex, nogosun")
     ap.add_argument("--design-context", type=int, default=2048, help="designs: tokens a decoding request holds")
     ap.add_argument("--workload", default="decode", choices=["decode", "mixed", "designs"],
                     help="decode: the default line; mixed: only the 0.6B-shaped mixed workload, as a line of its own")

@@ -7,6 +7,7 @@
 //   gelu (erf)     0.5 z (1 + erf(z / sqrt(2)))
 //   relu squared   max(z, 0)^2
 //   xIELU          z > 0: a z^2 + z/2;  z <= 0: b (e^z - 1 - z) + z/2
+// columns of a wider float32 tensor as rows of their own, rounded, with zeros behind them,
 // and the token shift: what a mixer reads of token t becomes x_t + (x_(t-1) - x_t) mix, the row before
 // a step's first token coming from the request's state.
 #include "common.h"
@@ -148,6 +149,18 @@ __global__ void rms_shift_kernel(const float* __restrict__ h, const TD* __restri
     }
 }
 
+// out[t, c] = x[t, column + c] for c < count, 0 for count <= c < size
+template <typename T>
+__global__ void columns_kernel(const float* __restrict__ x, int cols, int column, int count, T* __restrict__ out, int size,
+                               size_t total) {
+    for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
+         idx += (size_t)gridDim.x * blockDim.x) {
+        const size_t t = idx / size;
+        const int c = (int)(idx % size);
+        out[idx] = from_f32<T>(c < count ? x[t * cols + column + c] : 0.f);
+    }
+}
+
 static int blocks_for(size_t total) { return (int)((total + 255) / 256 < 8192 ? (total + 255) / 256 : 8192); }
 
 }  // namespace lc
@@ -268,5 +281,19 @@ LC_API int lc_bias_add(const void* x, int dt, const float* bias, void* out, int 
     else if (dt == DT_BF16) bias_add_kernel<bf16><<<blocks, 256, 0, stream>>>((const bf16*)x, bias, (bf16*)out, n, total);
     else LC_CHECK(false, "bias_add: unknown dtype %d", dt);
     LC_LAUNCH_CHECK("bias_add");
+    return 0;
+}
+
+// x float32 [T, cols] -> out [T, size] of dtype dt: its columns column .. column + count - 1, zeros behind them
+LC_API int lc_columns(const float* x, int cols, int column, int count, void* out, int dt, int T, int size,
+                      hipStream_t stream) {
+    LC_CHECK(T >= 0 && column >= 0 && count > 0 && column + count <= cols && size >= count, "columns: bad sizes");
+    if (T == 0) return 0;
+    LC_CHECK(x && out, "columns: null pointer");
+    const size_t total = (size_t)T * size;
+    if (dt == DT_F32) columns_kernel<float><<<blocks_for(total), 256, 0, stream>>>(x, cols, column, count, (float*)out, size, total);
+    else if (dt == DT_BF16) columns_kernel<bf16><<<blocks_for(total), 256, 0, stream>>>(x, cols, column, count, (bf16*)out, size, total);
+    else LC_CHECK(false, "columns: unknown dtype %d", dt);
+    LC_LAUNCH_CHECK("columns");
     return 0;
 }

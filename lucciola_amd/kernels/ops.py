@@ -115,6 +115,7 @@ _SIGNATURES = {
     "lc_state_space_readout": "pppiipiipifipip",
     "lc_scaled_sum": "pifpifpqp",
     "lc_bias_add": "pippiip",
+    "lc_columns": "piiipiiip",
     "lc_attention_rows": "piiiiiii" + "pppf" + "piip" + "pfp" + "pppipi" + "p",
     "lc_mlstm_prepare": "piiippf" + "pippi" + "iiiifi" + "ppp" + "p",
     "lc_mlstm_readout": "ppfpiipfiiipip",
@@ -2267,6 +2268,18 @@ def bias_add(x: torch.Tensor, bias: torch.Tensor) -> torch.Tensor:
     out = torch.empty_like(x)
     if x.numel():
         _call("lc_bias_add", _ptr(x), _dt(x), _ptr(bias), _ptr(out), x.shape[0], x.shape[1], _stream())
+    return out
+
+
+def columns(x: torch.Tensor, column: int, count: int, size: int, out_dtype: torch.dtype) -> torch.Tensor:
+    """Columns ``column`` .. + ``count`` of float32 ``x`` as rows of their own, [T, ``size``] of ``out_dtype``, zeros behind
+    them."""
+    _need(x, "columns x", torch.float32, 2)
+    if column < 0 or count < 1 or column + count > x.shape[1] or size < count:
+        raise KernelError(f"columns: {count} columns from {column} on of {tuple(x.shape)} into rows of {size}")
+    out = torch.empty((x.shape[0], size), dtype=out_dtype, device=x.device)
+    if x.shape[0]:
+        _call("lc_columns", _ptr(x), x.shape[1], column, count, _ptr(out), _dt(out), x.shape[0], size, _stream())
     return out
 
 

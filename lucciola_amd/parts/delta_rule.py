@@ -40,7 +40,7 @@ from ..config.registry import MIXERS
 from ..kernels import ops
 from ..weights.loader import ParamDecl
 from .base import BuildContext, Part
-from .feed_forward import low_rank, stack_rows
+from .feed_forward import low_rank_outer, stack_rows
 
 
 def _f32(t: torch.Tensor) -> torch.Tensor:
@@ -167,21 +167,26 @@ class ChannelDelta(Part):
 
     def declare(self) -> Dict[str, ParamDecl]:
         nq, nk, nv = self.nkv * self.dk, self.nh * self.dk, self.nh * self.dv
-        # the inner sizes of the decay's and the gate's two matrices are whatever the checkpoint holds
+        # the inner sizes of the decay's and the gate's two matrices are whatever the checkpoint holds (a head's size
+        # where there is none)
         return {"q": ParamDecl((nq, self.H)), "q_conv": ParamDecl((nq, self.taps), role="vector"),
                 "k": ParamDecl((nq, self.H)), "k_conv": ParamDecl((nq, self.taps), role="vector"),
                 "v": ParamDecl((nv, self.H)), "v_conv": ParamDecl((nv, self.taps), role="vector"),
                 "beta": ParamDecl((self.nh, self.H)), "rate_log": ParamDecl((self.nh,), role="vector"),
-                "rate_in": ParamDecl((-1, self.H)), "rate_out": ParamDecl((nk, -1)),
+                "rate_in": ParamDecl((-1, self.H), free_size=self.dk),
+                "rate_out": ParamDecl((nk, -1), free_size=self.dk),
                 "rate_bias": ParamDecl((nk,), role="vector"),
-                "gate_in": ParamDecl((-1, self.H)), "gate_out": ParamDecl((nv, -1)),
+                "gate_in": ParamDecl((-1, self.H), free_size=self.dv),
+                "gate_out": ParamDecl((nv, -1), free_size=self.dv),
                 "norm": ParamDecl((self.dv,), role="vector", init="ones_plus_normal"), "o": ParamDecl((self.H, nv))}
 
     def bind(self, tensors, ctx: BuildContext) -> None:
         self.dtype = ctx.dtype
-        self.proj = stack_rows([tensors[k] for k in ("q", "k", "v", "beta")])
-        self.inner, self.outer = low_rank((tensors["rate_in"], tensors["gate_in"]),
-                                          (tensors["rate_out"], tensors["gate_out"]), ctx.dtype == torch.bfloat16)
+        # the inner products of the decay and the gate ride along in the projection
+        inner = (tensors["rate_in"], tensors["gate_in"])
+        self.proj = stack_rows([tensors[k] for k in ("q", "k", "v")] + [*inner, tensors["beta"]])
+        self.rank = sum(t.shape[0] for t in inner)
+        self.outer = low_rank_outer(inner, (tensors["rate_out"], tensors["gate_out"]), ctx.dtype == torch.bfloat16)
         self.conv = torch.cat([_f32(tensors[k]) for k in ("q_conv", "k_conv", "v_conv")], dim=0).contiguous()
         self.rate_log, self.rate_bias = _f32(tensors["rate_log"]), _f32(tensors["rate_bias"])
         self.norm, self.o = _f32(tensors["norm"]), tensors["o"]
@@ -194,8 +199,9 @@ class ChannelDelta(Part):
         state, tail = site.cache
         proj = ops.gemm(x, self.proj, torch.float32)
         # columns: the decay's inputs, head by head and channel by channel, then the output gate's
-        gates = ops.gemm(ops.gemm(x, self.inner, self.dtype), self.outer, torch.float32)
-        coef, v = ops.channel_delta_prepare(proj, self.channels, gates, 0, tail, self.conv, self.rate_log,
+        inner = ops.columns(proj, self.channels, self.rank, self.outer.shape[1], self.dtype)
+        gates = ops.gemm(inner, self.outer, torch.float32)
+        coef, v = ops.channel_delta_prepare(proj, self.channels + self.rank, gates, 0, tail, self.conv, self.rate_log,
                                             self.rate_bias, self.nh, self.nkv, self.dk, self.dv, self.taps,
                                             self.unit_eps, batch.tok_req, batch.q_offsets, batch.slot_ids)
         ops.conv_tail_update(proj, tail, self.channels, self.taps, batch.q_offsets, batch.slot_ids,

@@ -23,24 +23,21 @@ def _softplus(z: float) -> float:
 INNER_MULTIPLE = 128        # what the matrix-core products want of a product's inner size
 
 
-def low_rank(inner, outer, pad: bool):
-    """Several pairs of small matrices, outer_k (inner_k x), as two products: the inner matrices stacked, and the outer
-    ones on the diagonal of one matrix (zeros elsewhere).  ``pad``: zero rows bring the inner size to a multiple of
-    INNER_MULTIPLE.  -> (inner [r, n], outer [sum of outer rows, r])"""
+def low_rank_outer(inner, outer, pad: bool):
+    """Several pairs of small matrices, outer_k (inner_k x), whose inner products stand side by side: the outer ones on the
+    diagonal of one matrix (zeros elsewhere), so that one product takes them all.  ``pad``: zero columns bring the inner
+    size to a multiple of INNER_MULTIPLE.  -> [sum of outer rows, r]"""
     for a, b in zip(inner, outer):
         if b.shape[1] != a.shape[0]:
             raise ValueError(f"the two matrices of a low-rank product do not fit each other ({tuple(a.shape)}, {tuple(b.shape)})")
     rank = sum(a.shape[0] for a in inner)
     size = -(-rank // INNER_MULTIPLE) * INNER_MULTIPLE if pad else rank
-    first = stack_rows(list(inner))
-    second = first.new_zeros((sum(b.shape[0] for b in outer), size))
+    out = outer[0].new_zeros((sum(b.shape[0] for b in outer), size))
     row = column = 0
     for b in outer:
-        second[row:row + b.shape[0], column:column + b.shape[1]] = b.to(second.dtype)
+        out[row:row + b.shape[0], column:column + b.shape[1]] = b.to(out.dtype)
         row, column = row + b.shape[0], column + b.shape[1]
-    if size > rank:
-        first = torch.cat([first, first.new_zeros((size - rank, first.shape[1]))]).contiguous()
-    return first, second
+    return out
 
 
 def stack_rows(tensors):

@@ -23,7 +23,7 @@ from ..config.registry import MIXERS
 from ..kernels import ops
 from ..weights.loader import ParamDecl
 from .base import BuildContext, Part
-from .feed_forward import low_rank, stack_rows
+from .feed_forward import low_rank_outer, stack_rows
 
 
 @MIXERS.register("gated_linear")
@@ -49,8 +49,11 @@ class GatedLinear(Part):
 
     def bind(self, tensors, ctx: BuildContext) -> None:
         self.dtype = ctx.dtype
-        self.proj = stack_rows([tensors[k] for k in ("q", "k", "v", "gate")])
-        self.inner, self.outer = low_rank((tensors["rate_in"],), (tensors["rate_out"],), ctx.dtype == torch.bfloat16)
+        # the decay's inner product rides along in the projection
+        self.proj = stack_rows([tensors[k] for k in ("q", "k", "v", "gate", "rate_in")])
+        self.gate_column = self.nh * (2 * self.dk + self.dv)
+        self.rank_column, self.rank = self.gate_column + self.nh * self.dv, tensors["rate_in"].shape[0]
+        self.outer = low_rank_outer((tensors["rate_in"],), (tensors["rate_out"],), ctx.dtype == torch.bfloat16)
         self.rate_bias, self.norm = (tensors[k].to(torch.float32).contiguous() for k in ("rate_bias", "norm"))
         self.o = tensors["o"]
 
@@ -61,11 +64,11 @@ class GatedLinear(Part):
         batch = site.batch
         (state,) = site.cache
         proj = ops.gemm(x, self.proj, torch.float32)
-        rates = ops.gemm(ops.gemm(x, self.inner, self.dtype), self.outer, torch.float32)
+        inner = ops.columns(proj, self.rank_column, self.rank, self.outer.shape[1], self.dtype)
+        rates = ops.gemm(inner, self.outer, torch.float32)
         coef, v = ops.gated_linear_prepare(proj, rates, 0, self.rate_bias, 1.0 / self.tau, self.dk ** -0.5, self.nh,
                                            self.dk, self.dv)
         o = ops.delta_scan(coef, v, state, batch.q_offsets, batch.slot_ids, batch.num_requests, self.nh, self.dk,
                            self.dv)
-        y = ops.head_gate_norm(o, proj, 2 * self.nh * self.dk + self.nh * self.dv, self.norm, False, self.norm_eps,
-                               "silu", self.nh, self.dv, self.dtype)
+        y = ops.head_gate_norm(o, proj, self.gate_column, self.norm, False, self.norm_eps, "silu", self.nh, self.dv, self.dtype)
         return ops.gemm(y, self.o, self.dtype, defer=True)

@@ -706,6 +706,12 @@ def scaled_sum(a, a_scale, b, b_scale):
     return (a_scale * a.to(F64) + b_scale * b.to(F64)).to(torch.float32)
 
 
+def columns(x, column, count, size, out_dtype):
+    out = torch.zeros(x.shape[0], size, dtype=out_dtype)
+    out[:, :count] = x[:, column:column + count].to(out_dtype)
+    return out
+
+
 def bias_add(x, bias):
     return (x.to(F64) + bias.to(F64)).to(x.dtype)
 
@@ -818,7 +824,7 @@ ALL = ("layer_norm", "layer_norm_act", "embedding_sinusoid", "gated_activation",
        "scale_", "token_shift", "rms_shift", "moe_route_sigmoid", "lightning_prepare", "lightning_readout",
        "gated_activation_weighted", "attention_prepare", "masked_attention", "state_space_prepare",
        "state_space_readout", "scaled_sum", "bias_add", "attention_rows", "mlstm_prepare", "mlstm_readout",
-       "attention_heads", "channel_delta_prepare", "gated_linear_prepare", "stream_norms")
+       "attention_heads", "channel_delta_prepare", "gated_linear_prepare", "stream_norms", "columns")
 
 
 def install(monkeypatch):

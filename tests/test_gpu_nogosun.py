@@ -346,6 +346,14 @@ def test_channel_delta_kernels(case_):
             assert float(states[DEV][0][slot].abs().max()) == 0.0
 
 
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("T,cols,column,count,size", [(1, 40, 3, 16, 128), (37, 300, 44, 256, 256), (2048, 131, 130, 1, 5)])
+def test_columns(dtype, T, cols, column, count, size):
+    x = torch.randn(T, cols, generator=torch.Generator().manual_seed(T))
+    assert torch.equal(ops.columns(x.to(DEV), column, count, size, dtype).cpu(),
+                       reference_ops.columns(x, column, count, size, dtype))
+
+
 @pytest.mark.parametrize("heads,dk,dv,tau", [(6, 32, 64, 16.0), (3, 7, 5, 1.0), (1, 128, 128, 4.0), (2, 256, 8, 100.0)])
 def test_gated_linear_kernels(heads, dk, dv, tau):
     g = torch.Generator().manual_seed(dk)

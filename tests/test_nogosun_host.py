@@ -27,7 +27,7 @@ from lucciola_amd.kernels import ops
 from lucciola_amd.models.causal_lm import declared_tensors
 from lucciola_amd.models.nogosun import nogosun_model_spec
 from lucciola_amd.parts.delta_rule import ChannelDelta
-from lucciola_amd.parts.feed_forward import RoutedMLP, low_rank
+from lucciola_amd.parts.feed_forward import RoutedMLP, low_rank_outer
 from lucciola_amd.parts.gated_linear import GatedLinear
 from lucciola_amd.parts.masked_attention import MaskedAttention
 from lucciola_amd.sampling.sampler import SamplingParams
@@ -196,7 +196,7 @@ def test_parts_refuse_what_no_kernel_has():
     with pytest.raises(ValueError, match="no kernel"):
         RoutedMLP(8, 8, 2, 1, activation="silu")
     with pytest.raises(ValueError, match="do not fit each other"):
-        low_rank((torch.zeros(3, 8),), (torch.zeros(5, 4),), False)
+        low_rank_outer((torch.zeros(3, 8),), (torch.zeros(5, 4),), False)
 
 
 def test_low_rank_products_on_one_diagonal():
@@ -205,9 +205,10 @@ def test_low_rank_products_on_one_diagonal():
     x = torch.randn(7, 8, generator=g)
     want = torch.cat([x @ a1.T @ a2.T, x @ b1.T @ b2.T], dim=1)
     for pad, rank in ((False, 7), (True, 128)):
-        inner, outer = low_rank((a1, b1), (a2, b2), pad)
-        assert inner.shape == (rank, 8) and outer.shape == (11, rank)
-        assert torch.allclose(x @ inner.T @ outer.T, want, atol=1e-5)
+        outer = low_rank_outer((a1, b1), (a2, b2), pad)
+        assert outer.shape == (11, rank)
+        inner = reference_ops.columns(torch.cat([x, x @ a1.T, x @ b1.T], dim=1), 8, 7, rank, torch.float32)
+        assert torch.allclose(inner @ outer.T, want, atol=1e-5)
 
 
 def test_branches_that_wait_together(monkeypatch):
