@@ -461,9 +461,9 @@ def nogosun_design_config(name, routed=True):
     width, heads, ff = DESIGN_SIZES[name]
     kv = max(1, heads // 4)
     moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 32, "top": 4}}
-    both = {"left": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+    both = {"left": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 25.0,
                      "q_temp": {"coef": 0.3, "every": 1024}},
-            "right": {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0}, "left_scale": 1.1, "right_scale": 0.9}
+            "right": {"heads": heads, "dim": 128, "vdim": 128, "tau": 8.0}, "left_scale": 1.1, "right_scale": 0.8}
     attention = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
                  "mask": {"size": 4096, "keep_first": 4},
                  "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}

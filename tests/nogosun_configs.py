@@ -66,7 +66,7 @@ N_B = {"architecture": "Nogosun", "vocab": 131, "width": 50, "norm": {"eps": 3e-
 # one over several pages
 _C = [
     layer(attention(8, 2, 32, 0.18, 20, 37, rot_dims=16, base=100000.0, stretch=(4.0, 64, 32.0, 1.0)), 128, 8, 2),
-    layer(parallel((8, 2, 64, 32, 0.125, 12.0, 0.5, 32), (4, 32, 64, 16.0), 1.2, 0.9), 64, 16, 4),
+    layer(parallel((8, 2, 64, 32, 0.125, 12.0, 0.6, 32), (4, 32, 64, 12.0), 1.3, 0.8), 64, 16, 4),
     layer(channel_delta(4, 2, 64, 32, 4), 128, 4, 2),
 ]
 _C += [borrows(_C, 1), borrows(_C, 2), layer(attention(4, 4, 64, 0.12, 50, 5, rot_dims=64, base=500.0), None)]
